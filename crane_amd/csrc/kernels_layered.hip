@@ -15,6 +15,8 @@ __device__ __forceinline__ float lay_act(float v, int act, float param = 1.f) {
     switch (act) {
         case LACT_RELU2: { const float r = fmaxf(v, 0.f); return r * r; }
         case LACT_LOGSIG: return param * (fminf(v, 0.f) - log1pf(expf(-fabsf(v))));      // ln sigmoid(v), no overflow either way
+        case LACT_SOFTPLUS: return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v)));
+        case LACT_SOFTCAP: return param * tanhf(v / param);
         case LACT_SILU: return v / (1.f + __expf(-v));
         case LACT_SIGMOID: return 1.f / (1.f + __expf(-v));
         case LACT_GELU_TANH: {
@@ -1965,7 +1967,8 @@ __device__ __forceinline__ void lay_router_choose(float* zs, int t, int lane, in
         bv = v;
         return at;
     };
-    // scores; the choice goes by score + correction (plain sigmoid scores: by the logits themselves, the same order)
+    // scores; the choice goes by score + correction (plain sigmoid scores: by the logits themselves, the same order -- unless groups are
+    // compared by sums of scores)
     if (rs.softmax) {
         float mx = -INFINITY;
         for (int ex = lane; ex < E; ex += 64) mx = fmaxf(mx, zs[ex]);
@@ -1976,16 +1979,20 @@ __device__ __forceinline__ void lay_router_choose(float* zs, int t, int lane, in
         for (int ex = lane; ex < E; ex += 64) sc[ex] /= sum;
     } else
         for (int ex = lane; ex < E; ex += 64) sc[ex] = 1.f / (1.f + expf(-zs[ex]));
-    if (rs.softmax || correction)
+    if (rs.softmax || correction || (rs.groups > 1 && rs.group_top > 1))
         for (int ex = lane; ex < E; ex += 64) zs[ex] = sc[ex] + (correction ? correction[ex] : 0.f);
     __builtin_amdgcn_wave_barrier();
     if (rs.groups > 1) {                   // keep the best groups: every pass removes the worst remaining one
         const int per = E / rs.groups;
-        float* gb = sc + E;                // [groups] a group's largest choice score (-inf: removed)
+        float* gb = sc + E;                // [groups] a group's score: its largest choice score, or the sum of its two largest (-inf: removed)
         for (int g = lane; g < rs.groups; g += 64) {
-            float best = -INFINITY;
-            for (int j = 0; j < per; ++j) best = fmaxf(best, zs[g * per + j]);
-            gb[g] = best;
+            float best = -INFINITY, second = -INFINITY;
+            for (int j = 0; j < per; ++j) {
+                const float v = zs[g * per + j];
+                second = fmaxf(second, fminf(best, v));
+                best = fmaxf(best, v);
+            }
+            gb[g] = rs.group_top > 1 && per > 1 ? best + second : best;
         }
         for (int drop = 0; drop < rs.groups - rs.keep_groups; ++drop) {
             // the worst live group, among equals the last one
@@ -2020,7 +2027,7 @@ __device__ __forceinline__ void lay_router_choose(float* zs, int t, int lane, in
         }
         __builtin_amdgcn_wave_barrier();
     }
-    for (int k = lane; k < top; k += 64) wsel[(size_t)t * slots + k] = rs.normalise ? wl[k] / (wsum + 1e-20f) : wl[k];
+    for (int k = lane; k < top; k += 64) wsel[(size_t)t * slots + k] = (rs.normalise ? wl[k] / (wsum + 1e-20f) : wl[k]) * rs.scale;
     for (int k = top + lane; k < slots; k += 64) wsel[(size_t)t * slots + k] = 1.f;
 }
 // logits and choice in one launch, one block per token

@@ -24,15 +24,16 @@ __device__ __forceinline__ float mx_softplus(float v) { return fmaxf(v, 0.f) + l
 // ------------------------------------------------------------------------------------------------------------------
 constexpr int LGN_MAX_GROUPS = 256;
 __global__ __launch_bounds__(256) void lay_add_gnorm_kernel(float* __restrict__ x, const int32_t* __restrict__ rows, const float* __restrict__ y,
-                                                            int nsum, const float* __restrict__ w, float* __restrict__ out, int W, int groups,
-                                                            float eps) {
+                                                            int nsum, const float* __restrict__ wsel, const float* __restrict__ w,
+                                                            float* __restrict__ out, int W, int groups, float eps) {
     __shared__ float rs[LGN_MAX_GROUPS];
     const int r = blockIdx.x, tid = threadIdx.x;
     float* xr = x + (size_t)(rows ? rows[r] : r) * W;
     if (y) {
         for (int c = tid; c < W; c += 256) {
             float v = xr[c];
-            for (int k = 0; k < nsum; ++k) v += y[((size_t)r * nsum + k) * W + c];      // fixed order: the same sum in every schedule
+            if (wsel) { for (int k = 0; k < nsum; ++k) v = fmaf(wsel[(size_t)r * nsum + k], y[((size_t)r * nsum + k) * W + c], v); }
+            else for (int k = 0; k < nsum; ++k) v += y[((size_t)r * nsum + k) * W + c];      // fixed order: the same sum in every schedule
             xr[c] = v;
         }
         if (!out) return;
@@ -49,10 +50,10 @@ __global__ __launch_bounds__(256) void lay_add_gnorm_kernel(float* __restrict__ 
     for (int c = tid; c < W; c += 256) out[(size_t)r * W + c] = xr[c] * rs[c / gw] * w[c];
 }
 void launch_lay_add_gnorm(float* x, const int32_t* rows, const float* y, int nsum, const float* w, float* out, int n_rows, int W, int groups,
-                          float eps, hipStream_t s) {
+                          float eps, hipStream_t s, const float* wsel) {
     if (n_rows <= 0 || (!y && !out)) return;
     if (groups <= 0 || groups > LGN_MAX_GROUPS || W % groups) groups = 1;       // the configuration reader has refused these
-    hipLaunchKernelGGL(lay_add_gnorm_kernel, dim3((unsigned)n_rows), dim3(256), 0, s, x, rows, y, nsum, w, out, W, groups, eps);
+    hipLaunchKernelGGL(lay_add_gnorm_kernel, dim3((unsigned)n_rows), dim3(256), 0, s, x, rows, y, nsum, wsel, w, out, W, groups, eps);
 }
 
 // ------------------------------------------------------------------------------------------------------------------

@@ -23,6 +23,11 @@
 //     state-space mixer (short causal convolution with bias and SiLU, one decay per head and token from a softplus step size, keys
 //     and queries shared by groups of heads, skip term, gate before a grouped norm).  Mixture-of-experts feed-forwards whose expert
 //     weight multiplies the expert's INPUT, with a capped gated activation, plus a shared expert.
+//   Rirotar -- pre-norm layers (norm weights stored around zero), logits capped by a tanh.  Mixers: latent attention without positions
+//     (queries straight from the input, one cached latent per token, sliding window, a sink per head) and two gated delta rules
+//     (S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q; short convolutions in front of q, k and v, unit-length q and k), one
+//     with a decay per head, one with a decay per key channel from a low-rank pair.  Capped gated feed-forwards, dense or routed
+//     (sigmoid scores, the best groups by the sum of their two largest scores, weights divided by their sum and scaled).
 // The mechanisms are kernels with their constants as arguments (kernels_layered.hip); the per-layer plumbing and the step function
 // over mixed batches (prompt portions beside single decode tokens) are in model_layered.cpp.
 #pragma once
@@ -36,11 +41,13 @@ namespace cm {
 
 // LMIX_SIDE: the mixers in LayerSpec::side run side by side on the layer's input; LMIX_MEMORY: matrix memory with exponential gates
 // LMIX_HGRN: gated linear recurrence with k = 1 - forget gate; LMIX_SSM: state-space mixer (one decay per head and token)
-enum { LMIX_ATTN = 0, LMIX_LIGHTNING = 1, LMIX_LATENT = 2, LMIX_GLA = 3, LMIX_MEMORY = 4, LMIX_SIDE = 5, LMIX_HGRN = 6, LMIX_SSM = 7 };
+// LMIX_DELTA: gated delta rule
+enum { LMIX_ATTN = 0, LMIX_LIGHTNING = 1, LMIX_LATENT = 2, LMIX_GLA = 3, LMIX_MEMORY = 4, LMIX_SIDE = 5, LMIX_HGRN = 6, LMIX_SSM = 7, LMIX_DELTA = 8 };
 enum { LMLP_NONE = 0, LMLP_DENSE = 1, LMLP_MOE = 2 };
 // LACT_RELU2: max(v, 0)^2;  LACT_LOGSIG: act_param * ln(sigmoid(v)) (the logarithm of a decay sigmoid(v)^act_param)
 // LACT_CAPGLU (two-matrix products only): g = min(g, cap), u = clamp(u, -cap, cap): g sigmoid(1.702 g) (u + 1), cap = act_param
-enum { LACT_NONE = 0, LACT_SILU = 1, LACT_SIGMOID = 2, LACT_GELU_TANH = 3, LACT_RELU2 = 4, LACT_LOGSIG = 5, LACT_CAPGLU = 6 };
+// LACT_SOFTPLUS: ln(1 + e^v);  LACT_SOFTCAP: act_param * tanh(v / act_param)
+enum { LACT_NONE = 0, LACT_SILU = 1, LACT_SIGMOID = 2, LACT_GELU_TANH = 3, LACT_RELU2 = 4, LACT_LOGSIG = 5, LACT_CAPGLU = 6, LACT_SOFTPLUS = 7, LACT_SOFTCAP = 8 };
 // distance term taken off an attention score: none | r1 ln(1 + r2 (i - j)) | r1 (i - j)
 enum { LBIAS_NONE = 0, LBIAS_LOG = 1, LBIAS_LINEAR = 2 };
 // gate on the attention output: none | one value per head at g_off + head | one per element at g_off + head e + i
@@ -63,8 +70,10 @@ struct RotSpec {
 struct RouterSpec {
     bool softmax = false;              // scores: softmax over all outputs (false: sigmoid of each)
     bool correction = false;           // a learned vector joins the scores for the choice only
-    int groups = 1, keep_groups = 1;   // outputs form `groups` equal groups of neighbours; only the keep_groups best (by their largest choice score) can be chosen
+    int groups = 1, keep_groups = 1;   // outputs form `groups` equal groups of neighbours; only the keep_groups best can be chosen
+    int group_top = 1;                 // a group's score: the sum of its group_top (1 or 2) largest choice scores
     bool normalise = false;            // weights divided by their sum
+    float scale = 1.f;                 // ... then times this
     int identity = 0;                  // the last `identity` outputs pass the input through (no matrices)
 };
 
@@ -79,7 +88,8 @@ struct LayerSpec {
     int bias = LBIAS_NONE, gate = LGATE_NONE;
     bool sink = false, own_v = false;  // attention: learned sink per head in the softmax denominator; value projection of its own
     int kv_from = -1;                  // attention: keys and values of that earlier layer's cache instead of own projections
-    int q_rank = 0, kv_rank = 0, rot_dim = 0;   // latent attention
+    int q_rank = 0, kv_rank = 0, rot_dim = 0;   // latent attention (q_rank 0: queries straight from the input)
+    bool gate_latent = false;          // ... element-wise gate on the values after their up-projection
     RotSpec rot;
     float tau = 1.f;                   // gated linear attention: decay = sigmoid(z)^(1 / tau)
     int a_rank = 0;                    // ... inner size of the decay's low-rank projection (from the checkpoint)
@@ -104,6 +114,9 @@ struct LayerSpec {
     bool scale_input = false;          // mixture of experts: the expert's weight multiplies its input (false: its output)
     int expert_act = LACT_SILU; float limit = 0.f, shared_limit = 0.f;    // experts: activation of the gated product and its cap
     int weights_of = -1;               // the layer runs on that earlier layer's tensors, with a cache and state of its own
+    // delta rule (conv: taps of the convolutions on q, k, v): one decay per key channel (a low-rank pair, as the output gate) instead of
+    // one per head; g_rank: inner size of the output gate's pair (from the checkpoint, as a_rank)
+    bool channel_decay = false; int g_rank = 0;
 };
 
 // device-side weights of one layer (bf16 matrices [out, in], f32 vectors)
@@ -150,10 +163,15 @@ struct LayeredLayerW {
     float *conv_w = nullptr, *conv_b = nullptr, *dt_bias = nullptr, *a_neg = nullptr, *skip = nullptr;
     int z_off = 0, x_off = 0, dt_off = 0;
     size_t cv_off = 0;                               // the convolution's last taps - 1 inputs inside a slot of the conv pool (floats)
+    // delta rule: columns of the projection row: q_off: q | k | v (the convolution's channels) | b_off (write strength) | a_off (decay per head, or
+    // a1) | g_off (gate, or g1);  a2: [H d][a_rank], g2: [H e][g_rank];  conv_w, dt_bias ([H] or [H d]), a_neg ([H]), mix_norm ([e])
+    int b_off = 0;
+    uint16_t* g2 = nullptr;
     std::vector<LayeredLayerW> side;
 };
 
-// rows [row0, row0 + n) of a pass are positions start_pos.. of the sequence in `slot`; its page table starts at bt_off
+// rows [row0, row0 + n) of a pass are positions start_pos.. of the sequence in `slot`; its page table starts at bt_off.  pad0: its first
+// chunk of LAY_LIGHT_CHUNK tokens; pad1: its first chunk of LAY_DELTA_CHUNK tokens
 struct LaySegDev { int row0, n, start_pos, slot, bt_off, pad0, pad1, pad2; };
 
 struct LGemmArgs {
@@ -293,10 +311,11 @@ void launch_lay_rms_gate(const float* o, const float* gate, int ldg, const float
                          int group = 0, bool shared_w = false);
 
 // ---- kernels_layered_mix.hip ----
-// x[r] += sum_(k < nsum) y[(r nsum + k) W ..] (y null: nothing is added), then out[r] = x[rows ? rows[r] : r] in `groups` equal
-// consecutive parts, each over its own root mean square, times w (out null: the update alone).  rows and y exclude each other.
+// x[r] += sum_(k < nsum) y[(r nsum + k) W ..] (y null: nothing is added; wsel given: row k times wsel[r nsum + k]), then out[r] =
+// x[rows ? rows[r] : r] in `groups` equal consecutive parts, each over its own root mean square, times w (out null: the update alone).
+// rows and y exclude each other.
 void launch_lay_add_gnorm(float* x, const int32_t* rows, const float* y, int nsum, const float* w, float* out, int n_rows, int W, int groups,
-                          float eps, hipStream_t s);
+                          float eps, hipStream_t s, const float* wsel = nullptr);
 // two-map attention: a [T][2 H e] holds the maps' outputs, key head g's heads of map m at columns ((2 g + m) nrep + j) e; out[t][h e + i] =
 // unit_rms_e(a1 - lambda a2) * post
 void launch_lay_diff_combine(const float* a, float* out, int T, int H, int G, int e, float lambda, float post, float eps, hipStream_t s);
@@ -329,6 +348,38 @@ bool lay_attn_talk_fits(int H, int G, int d, int e);
 // value tiles), which also takes LAttnArgs::v_div
 void launch_lay_attn_talk_mfma(const LAttnArgs& a, const float* talk, int nseg, int max_n, hipStream_t s);
 bool lay_attn_talk_mfma_fits(int H, int G, int d, int e, int v_div = 1, bool mixed = true);
+
+// ---- kernels_layered_delta.hip ----
+// latent rows on their way into the cache, one launch: RMS norm of the columns [k_off, k_off + n) times w, into the pages [n_pages][page][n]
+void launch_lay_latent_append(const float* proj, int ldp, int k_off, int n, const float* w, float eps, void* kpool, int kvt, const int32_t* bt,
+                              const LaySegDev* segs, const int32_t* rowseg, int T, int page, hipStream_t s);
+// Gated delta rule, per head (state S [d][e] f32): S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q, and
+// out = o / rms_e(o) * norm_w * gate.  g = exp of one logarithm per head, or per head and key channel (channel).
+struct LDeltaArgs {
+    const float* proj; int ldp;                      // projection rows
+    int q_off, b_off, a_off;                         // q | k | v from q_off; write strengths (before the sigmoid); head form: decay inputs
+    int H, G, d, e;                                  // heads, query / key heads, key size, value size
+    const float* conv_w; int taps;                   // [2 G d + H e][taps]
+    float* conv_pool; size_t conv_stride, cv_off;    // tails [taps - 1][channels], oldest first
+    const float *dt_bias, *a_neg;                    // head form: ln g = a_neg[h] softplus(a + dt_bias[h]);  channel: ln g = a_neg[h] ldec
+    float* xb;                                       // [T][2 G d + H e]: convolved q (unit length, times d^(-1/2)) | k (unit length) | v
+    float* beta;                                     // [T][H]
+    float* ldec; bool channel;                       // [T][H] (written by the preparation), or [T][H d] (channel: softplus already applied)
+    float* state_pool; size_t slot_stride, st_off;
+    const LaySegDev* segs; const int32_t* rowseg; int nseg, T;
+    const float* gate; int ldg;                      // activated output gate [T][H e]
+    const float* norm_w; float eps;
+    float* o_raw;                                    // [T][H e] scratch (token-by-token form)
+    float* out;                                      // [T][H e]
+    bool all_single;                                 // every portion of the pass is one token
+    // chunk-parallel form for portions of more than LAY_DELTA_SEQ tokens: table {segment, first token}, segs[].pad1 = a segment's first
+    // chunk; scratch of lay_delta_chunk_floats per (chunk, head).  Null / 0: every portion token by token.
+    const int2* chunks = nullptr; int nchunks = 0; float* scratch = nullptr;
+};
+constexpr int LAY_DELTA_CHUNK = 64, LAY_DELTA_SEQ = 16;
+bool lay_delta_chunk_fits(int d, int e);             // sizes the chunk-parallel form takes
+size_t lay_delta_chunk_floats(int d, int e);
+void launch_lay_delta(const LDeltaArgs& a, hipStream_t s);
 
 // router: z = h . Wr^T in f32 over E outputs, scores by rs (sigmoid of each / softmax over all), the `top` largest choice scores
 // (score + correction, inside the best groups; lowest index first among equals) -> sel [T top], wsel [T slots] = their scores

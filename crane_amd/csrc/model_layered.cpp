@@ -7,8 +7,10 @@
 // continuing its sequence from the cache and state earlier steps left; forward / prefill_multi / decode_batch / generate and the
 // engine's scheduler all go through it for this family.
 #include <algorithm>
+#include <cctype>
 #include <cmath>
 #include <cstring>
+#include <iterator>
 #include <map>
 
 #include "json_min.h"
@@ -28,11 +30,18 @@ struct Layered {
     // Gibipel: a sublayer reads the residual itself and a one-number norm sits on its output; embedding and logits are scaled
     bool post_only = false;
     float embed_scale = 1.f, logit_scale = 1.f;
-    // Nevotar: x += mixer(norm1 x), x += ff(norm2 x); the norms work on norm_groups equal parts of the vector; the logits come from the
-    // embedding table
+    // Nevotar, Rirotar: x += mixer(norm1 x), x += ff(norm2 x).  Nevotar's norms work on norm_groups equal parts of the vector and its
+    // logits come from the embedding table; Rirotar's logits pass logit_cap tanh(z / logit_cap)
     bool pre_norm = false;
     int norm_groups = 1;
-    int max_conv = 0;                  // widest convolution of a state-space mixer (channels)
+    float logit_cap = 0.f;
+    std::string arch;
+    int max_conv = 0;                  // widest convolution of a state-space mixer or delta rule (channels)
+    int max_gt = 0;
+    float* GT = nullptr;               // [cap][max_gt] activated output gates from a low-rank pair
+    float* DS = nullptr;               // delta rules, chunk-parallel form: ds_chunks chunks of ds_stride floats
+    size_t ds_stride = 0;
+    int ds_chunks = 0;
     float* XB = nullptr;               // [cap][max_conv] convolved and activated channels
     int max_mh = 0, max_sff = 0, max_slots = 1;   // matrix-memory heads, shared expert size, rows per token of an expert combine
     float* Z = nullptr;                // router logits [cap][most outputs]
@@ -121,6 +130,7 @@ static void parse_mlp(const cmjson::Value* ml, LayerSpec& sp, bool moe_ok) {
     if (kind == "dense") {
         sp.mlp = LMLP_DENSE;
         sp.ff = (int)ml->integer("ff", 0);
+        sp.limit = (float)ml->number("limit", 0.0);
     } else if (kind == "moe" && moe_ok) {
         sp.mlp = LMLP_MOE;
         const cmjson::Value* ex = ml->get("expert");
@@ -131,6 +141,7 @@ static void parse_mlp(const cmjson::Value* ml, LayerSpec& sp, bool moe_ok) {
         sp.experts = (int)rt->integer("experts", 0);
         sp.top = (int)rt->integer("top", 0);
         sp.router.identity = (int)rt->integer("identity", 0);
+        sp.router.scale = (float)rt->number("scale", 1.0);
         if (const cmjson::Value* gr = rt->get("groups"))
             if (gr->kind == cmjson::Value::Obj) {
                 sp.router.groups = (int)gr->integer("count", 1);
@@ -228,6 +239,7 @@ static void parse_mononex_layer(const cmjson::Value& e, LayerSpec& sp, const std
         sp.scale = (float)mx->number("scale", 1.0 / std::sqrt((double)(sp.dim + sp.rot_dim)));
         sp.kv_heads = 1;               // one cached row per token: [latent | rotated key part]
         sp.gate = LGATE_NONE;          // the gate acts on the values after their up-projection
+        sp.gate_latent = true;
         if (const cmjson::Value* rt = mx->get("rot"))
             if (rt->kind == cmjson::Value::Obj) {
                 sp.rot.dims = (int)rt->integer("dims", sp.rot_dim);
@@ -422,18 +434,67 @@ static void parse_nevotar_layer(const cmjson::Value& e, LayerSpec& sp, const std
         }
 }
 
+// Rirotar: layer types "latent_attention" ("heads", "dim", "vdim", "kv_rank", "scale", "mask": {"size"}), "delta" and "channel_delta"
+// ("heads", "kv_heads", "dim", "vdim", "conv"); "mlp": {"kind": "dense", "ff", "limit"} or {"kind": "moe", "expert": {"ff", "limit"},
+// "router": {"experts", "top", "groups": {"count", "keep"}, "scale"}}
+static void parse_rirotar_layer(const cmjson::Value& e, LayerSpec& sp) {
+    const std::string type = e.string("type", "");
+    const cmjson::Value* mx = e.get("mixer");
+    need(mx && mx->kind == cmjson::Value::Obj, "layer without mixer");
+    sp.heads = (int)mx->integer("heads", 0);
+    sp.dim = (int)mx->integer("dim", 0);
+    sp.vdim = (int)mx->integer("vdim", sp.dim);
+    need(sp.heads > 0 && sp.dim > 0 && sp.vdim > 0, "mixer sizes");
+    sp.win = 1ll << 40; sp.keep = 0;
+    sp.gate = LGATE_NONE;
+    if (type == "latent_attention") {
+        sp.mixer = LMIX_LATENT;
+        sp.kv_heads = 1;               // one cached row per token: the latent
+        sp.kv_rank = (int)mx->integer("kv_rank", 0);
+        need(sp.kv_rank > 0, "kv_rank");
+        sp.scale = (float)mx->number("scale", 1.0 / std::sqrt((double)sp.dim));
+        sp.sink = true;
+        if (const cmjson::Value* mk = mx->get("mask"))
+            if (mk->kind == cmjson::Value::Obj) {
+                sp.win = mk->integer("size", sp.win);
+                need(sp.win > 0, "mask.size");
+            }
+        need(lay_attn_fits(sp.kv_rank, sp.kv_rank, false), "kv_rank too large");
+    } else if (type == "delta" || type == "channel_delta") {
+        sp.mixer = LMIX_DELTA;
+        sp.channel_decay = type == "channel_delta";
+        sp.kv_heads = (int)mx->integer("kv_heads", sp.heads);
+        sp.conv = (int)mx->integer("conv", 1);
+        need(sp.kv_heads > 0 && sp.heads % sp.kv_heads == 0, "heads % kv_heads != 0");
+        need(sp.conv >= 1 && sp.conv <= 64, "conv");
+        if (sp.dim > 256) throw CmError(CM_ERR_UNSUPPORTED, "delta rule key size above 256");
+    } else throw CmError(CM_ERR_UNSUPPORTED, "layer type '" + type + "' not implemented");
+    parse_mlp(e.get("mlp"), sp, true);
+    sp.ff_act = sp.expert_act = LACT_CAPGLU;
+    need(sp.mlp == LMLP_NONE || sp.limit > 0.f, "mlp limit");
+    need(sp.router.identity == 0 && sp.shared_ff == 0, "router.identity / shared are not part of this design");
+    sp.router.group_top = 2; sp.router.normalise = true;
+}
+
 // config.json of a layer-list decoder: "architecture", "vocab", "width", "norm".eps and "layers": [{"type", "mixer": {...}, "mlp"}]
 void Model::init_layered_config(const cmjson::Value& root) {
     const std::string arch = root.string("architecture", "");
-    if (arch != "Korupel" && arch != "Mononex" && arch != "Gibipel" && arch != "Nevotar")
-        throw CmError(CM_ERR_UNSUPPORTED, "architecture '" + arch + "' not implemented (Korupel, Mononex, Gibipel, Nevotar)");
+    const char* known[] = {"Korupel", "Mononex", "Gibipel", "Nevotar", "Rirotar"};
+    if (std::find(std::begin(known), std::end(known), arch) == std::end(known))
+        throw CmError(CM_ERR_UNSUPPORTED, "architecture '" + arch + "' not implemented (Korupel, Mononex, Gibipel, Nevotar, Rirotar)");
     layered = true;
     lay.reset(new Layered());
     Layered& L = *lay;
+    L.arch = arch;
     L.parallel = arch == "Mononex";
     L.post_only = arch == "Gibipel";
-    L.pre_norm = arch == "Nevotar";
-    cfg.model_type = L.parallel ? "mononex" : (L.post_only ? "gibipel" : (L.pre_norm ? "nevotar" : "korupel"));
+    L.pre_norm = arch == "Nevotar" || arch == "Rirotar";
+    cfg.model_type = arch;
+    for (char& c : cfg.model_type) c = (char)std::tolower((unsigned char)c);
+    if (arch == "Rirotar") {
+        L.logit_cap = (float)root.number("logit_softcap", 0.0);
+        need(L.logit_cap > 0.f, "logit_softcap");
+    }
     if (L.post_only) {
         if (const cmjson::Value* em = root.get("embedding")) L.embed_scale = (float)em->number("scale", 1.0);
         L.logit_scale = (float)root.number("logit_scale", 1.0);
@@ -442,7 +503,7 @@ void Model::init_layered_config(const cmjson::Value& root) {
     cfg.H = (int)root.integer("width", 0);
     if (const cmjson::Value* n = root.get("norm")) {
         cfg.eps = (float)n->number("eps", 1e-6);
-        if (L.pre_norm) L.norm_groups = (int)n->integer("groups", 1);
+        if (arch == "Nevotar") L.norm_groups = (int)n->integer("groups", 1);
     }
     if (!L.parallel && !L.post_only && !L.pre_norm) {
         if (const cmjson::Value* c = root.get("canon")) L.taps = (int)c->integer("taps", 0);
@@ -457,7 +518,8 @@ void Model::init_layered_config(const cmjson::Value& root) {
         LayerSpec sp;
         if (L.parallel) parse_mononex_layer(*e, sp, L.spec);
         else if (L.post_only) parse_gibipel_layer(*e, sp);
-        else if (L.pre_norm) parse_nevotar_layer(*e, sp, L.spec);
+        else if (arch == "Nevotar") parse_nevotar_layer(*e, sp, L.spec);
+        else if (arch == "Rirotar") parse_rirotar_layer(*e, sp);
         else parse_korupel_layer(*e, sp);
         L.spec.push_back(sp);
     }
@@ -584,12 +646,14 @@ static std::vector<float> rot_frequencies(const RotSpec& r, float* mag) {
 static void build_mononex(Model& m, LaySource& src);
 static void build_gibipel(Model& m, LaySource& src);
 static void build_nevotar(Model& m, LaySource& src);
+static void build_rirotar(Model& m, LaySource& src);
 
 static void build_layered(Model& m, LaySource& src) {
     Layered& L = *m.lay;
     if (L.parallel) { build_mononex(m, src); return; }
     if (L.post_only) { build_gibipel(m, src); return; }
-    if (L.pre_norm) { build_nevotar(m, src); return; }
+    if (L.arch == "Nevotar") { build_nevotar(m, src); return; }
+    if (L.arch == "Rirotar") { build_rirotar(m, src); return; }
     const size_t W = (size_t)m.cfg.H, V = (size_t)m.cfg.V;
     const float ws = 1.0f / std::sqrt((float)W);
     m.embed = up_bf16(m, src.get("embed", V * W, 1.0f, 0.f));
@@ -660,6 +724,18 @@ static void build_layered(Model& m, LaySource& src) {
 // norm weights stored around zero: the factor is 1 + w
 static std::vector<float> plus_one(std::vector<float> v) { for (float& x : v) x += 1.f; return v; }
 
+// up-projections of a cached latent.  W_uk per head, transposed: the product q . (W_uk c) = (W_uk^T q) . c runs against the cached latent
+static void build_latent_up(Model& m, LaySource& src, const std::string& p, const LayerSpec& sp, LayeredLayerW& w) {
+    const size_t H = (size_t)sp.heads, d = (size_t)sp.dim, e = (size_t)sp.vdim, kr = (size_t)sp.kv_rank;
+    const std::vector<float> uk = src.get(p + "mix.uk", H * d * kr, 1.0f / std::sqrt((float)kr), 0.f);
+    std::vector<float> t(H * kr * d);
+    for (size_t h = 0; h < H; ++h)
+        for (size_t a = 0; a < d; ++a)
+            for (size_t c = 0; c < kr; ++c) t[(h * kr + c) * d + a] = uk[(h * d + a) * kr + c];
+    w.uk_t = up_bf16(m, t);
+    w.uv = up_bf16(m, src.get(p + "mix.uv", H * e * kr, 1.0f / std::sqrt((float)kr), 0.f));
+}
+
 static void build_mononex(Model& m, LaySource& src) {
     Layered& L = *m.lay;
     const size_t W = (size_t)m.cfg.H, V = (size_t)m.cfg.V;
@@ -705,15 +781,7 @@ static void build_mononex(Model& m, LaySource& src) {
             w.dq_norm = up_f32(m, src.get(p + "mix.dq.norm", qr, 0.1f, 1.f));
             w.dkv_norm = up_f32(m, src.get(p + "mix.dkv.norm", kr, 0.1f, 1.f));
             w.uq = up_bf16(m, src.get(p + "mix.uq", H * (d + r) * qr, 1.0f / std::sqrt((float)qr), 0.f));
-            {   // W_uk per head, transposed: the product q_unrotated . (W_uk c) = (W_uk^T q_unrotated) . c runs against the cached latent
-                const std::vector<float> uk = src.get(p + "mix.uk", H * d * kr, 1.0f / std::sqrt((float)kr), 0.f);
-                std::vector<float> t(H * kr * d);
-                for (size_t h = 0; h < H; ++h)
-                    for (size_t a = 0; a < d; ++a)
-                        for (size_t c = 0; c < kr; ++c) t[(h * kr + c) * d + a] = uk[(h * d + a) * kr + c];
-                w.uk_t = up_bf16(m, t);
-            }
-            w.uv = up_bf16(m, src.get(p + "mix.uv", H * e * kr, 1.0f / std::sqrt((float)kr), 0.f));
+            build_latent_up(m, src, p, sp, w);
             if (sp.rot.dims > 0) w.rot_freq = up_f32(m, rot_frequencies(sp.rot, &w.rot_mag));
             w.o_w = up_bf16(m, src.get(p + "mix.o", W * H * e, 1.0f / std::sqrt((float)(H * e)), 0.f));
             w.kv_idx = kv_idx++;
@@ -970,6 +1038,82 @@ static void build_nevotar(Model& m, LaySource& src) {
     m.lm_head = L.head;
 }
 
+static void build_rirotar(Model& m, LaySource& src) {
+    Layered& L = *m.lay;
+    const size_t W = (size_t)m.cfg.H, V = (size_t)m.cfg.V;
+    const float ws = 1.0f / std::sqrt((float)W);
+    m.embed = up_bf16(m, src.get("embed", V * W, 1.0f, 0.f));
+    L.w.resize(L.spec.size());
+    for (size_t i = 0; i < L.spec.size(); ++i) {
+        LayerSpec& sp = L.spec[i];
+        LayeredLayerW& w = L.w[i];
+        const std::string p = "l" + std::to_string(i) + ".", q = p + "mix.";
+        const size_t H = (size_t)sp.heads, G = (size_t)sp.kv_heads, d = (size_t)sp.dim, e = (size_t)sp.vdim;
+        w.norm1 = up_f32(m, plus_one(src.get(p + "norm1", W, 0.1f, 0.f)));
+        std::vector<float> in;
+        if (sp.mixer == LMIX_LATENT) {         // q | latent
+            const size_t kr = (size_t)sp.kv_rank;
+            w.q_off = 0; w.k_off = (int)(H * d); w.g_off = w.k_off + (int)kr;
+            append(in, src.get(q + "q", H * d * W, ws, 0.f));
+            append(in, src.get(q + "dkv", kr * W, ws, 0.f));
+            w.dkv_norm = up_f32(m, src.get(q + "dkv.norm", kr, 0.1f, 1.f));
+            build_latent_up(m, src, p, sp, w);
+            w.sink = up_f32(m, src.get(q + "sink", H, 1.0f, 0.f));
+        } else {                               // q | k | v | write strength | decay | gate;  channel form: q | k | v | a1 | g1 | write strength
+            const size_t C = 2 * G * d + H * e, taps = (size_t)sp.conv;
+            const float cs = 1.0f / std::sqrt((float)taps);
+            std::vector<float> cw, an = src.get(q + "A_log", H, 0.5f, 0.f);
+            w.q_off = 0; w.k_off = (int)(G * d); w.v_off = (int)(2 * G * d);
+            for (const char* n : {"q", "k", "v"}) {
+                const size_t rows = *n == 'v' ? H * e : G * d;
+                append(in, src.get(q + n, rows * W, ws, 0.f));
+                append(cw, src.get(q + n + ".conv", rows * taps, cs, 0.f));
+            }
+            w.conv_w = up_f32(m, cw);
+            for (float& v : an) v = (float)(-std::exp((double)v));
+            w.a_neg = up_f32(m, an);
+            if (sp.channel_decay) {
+                sp.a_rank = (int)src.dim0(q + "a1", 32);
+                sp.g_rank = (int)src.dim0(q + "g1", 32);
+                if (sp.a_rank <= 0 || sp.g_rank <= 0) throw CmError(CM_ERR_IO, "tensor " + q + "a1 / g1: unexpected shape");
+                const size_t ar = (size_t)sp.a_rank, gr = (size_t)sp.g_rank;
+                w.a_off = (int)C; w.g_off = w.a_off + (int)ar; w.b_off = w.g_off + (int)gr;
+                append(in, src.get(q + "a1", ar * W, ws, 0.f));
+                append(in, src.get(q + "g1", gr * W, ws, 0.f));
+                append(in, src.get(q + "b", H * W, ws, 0.f));
+                w.a2 = up_bf16(m, src.get(q + "a2", H * d * ar, 1.0f / std::sqrt((float)ar), 0.f));
+                w.g2 = up_bf16(m, src.get(q + "g2", H * e * gr, 1.0f / std::sqrt((float)gr), 0.f));
+                w.dt_bias = up_f32(m, src.get(q + "dt_bias", H * d, 0.5f, -3.f));
+            } else {
+                w.b_off = (int)C; w.a_off = w.b_off + (int)H; w.g_off = w.a_off + (int)H;
+                append(in, src.get(q + "b", H * W, ws, 0.f));
+                append(in, src.get(q + "a", H * W, ws, 0.f));
+                append(in, src.get(q + "g", H * e * W, ws, 0.f));
+                w.dt_bias = up_f32(m, src.get(q + "dt_bias", H, 0.5f, -3.f));
+            }
+            w.mix_norm = up_f32(m, src.get(q + "norm", e, 0.1f, 1.f));
+        }
+        // whole tiles for the projection's kernels: rows of zeros behind the last one (their products are not read)
+        const size_t rows = in.size() / W, unit = rows >= 1024 ? 128 : 8;
+        w.in_rows = (int)((rows + unit - 1) / unit * unit);
+        in.resize((size_t)w.in_rows * W, 0.f);
+        w.in_w = up_bf16(m, in);
+        w.o_w = up_bf16(m, src.get(q + "o", W * H * e, 1.0f / std::sqrt((float)(H * e)), 0.f));
+        if (sp.mlp == LMLP_NONE) continue;
+        w.norm2 = up_f32(m, plus_one(src.get(p + "norm2", W, 0.1f, 0.f)));
+        if (sp.mlp == LMLP_MOE) build_experts(m, src, p, sp, w);
+        else {
+            const size_t ff = (size_t)sp.ff;
+            w.gate = up_bf16(m, src.get(p + "mlp.gate", ff * W, ws, 0.f));
+            w.up = up_bf16(m, src.get(p + "mlp.up", ff * W, ws, 0.f));
+            w.down = up_bf16(m, src.get(p + "mlp.down", W * ff, 1.0f / std::sqrt((float)ff), 0.f));
+        }
+    }
+    L.final_norm = up_f32(m, plus_one(src.get("final.norm", W, 0.1f, 0.f)));
+    L.head = up_bf16(m, src.get("head", V * W, ws, 0.f));
+    m.lm_head = L.head;
+}
+
 void load_layered_from_dir(Model& m, const std::string& dir) {
     try {
         LayFileSource src(dir);
@@ -1045,7 +1189,7 @@ void Model::alloc_runtime_layered() {
             if (sp.mixer == LMIX_LATENT) {
                 L.max_o = std::max(L.max_o, sp.heads * sp.vdim);
                 L.max_cq = std::max(L.max_cq, sp.q_rank);
-                L.max_q = std::max(L.max_q, sp.heads * (sp.dim + sp.rot_dim));
+                if (sp.q_rank > 0) L.max_q = std::max(L.max_q, sp.heads * (sp.dim + sp.rot_dim));
                 L.max_qa = std::max(L.max_qa, sp.heads * dk);
             }
         } else if (sp.mixer == LMIX_MEMORY) {
@@ -1066,6 +1210,19 @@ void Model::alloc_runtime_layered() {
             L.max_o = std::max(L.max_o, sp.heads * sp.vdim);
             L.max_ld = std::max(L.max_ld, sp.heads);
             L.max_mh = std::max(L.max_mh, sp.heads);
+        } else if (sp.mixer == LMIX_DELTA) {
+            // state [H][d][e]; the convolutions' last taps - 1 inputs [taps - 1][q | k | v]
+            w.st_off = st;
+            st += (size_t)sp.heads * sp.dim * sp.vdim;
+            const int C = 2 * sp.kv_heads * sp.dim + sp.heads * sp.vdim;
+            w.cv_off = cv;
+            cv += (size_t)(sp.conv - 1) * C;
+            L.max_conv = std::max(L.max_conv, C);
+            L.max_o = std::max(L.max_o, sp.heads * sp.vdim);
+            L.max_ld = std::max(L.max_ld, sp.heads * (sp.channel_decay ? sp.dim : 1));
+            L.max_mh = std::max(L.max_mh, sp.heads);
+            if (sp.channel_decay) L.max_gt = std::max(L.max_gt, sp.heads * sp.vdim);
+            if (lay_delta_chunk_fits(sp.dim, sp.vdim)) L.ds_stride = std::max(L.ds_stride, (size_t)sp.heads * lay_delta_chunk_floats(sp.dim, sp.vdim));
         } else {
             w.st_off = st;
             st += (size_t)sp.heads * sp.dim * sp.vdim;
@@ -1126,7 +1283,12 @@ void Model::alloc_runtime_layered() {
     if (L.max_cq) {
         L.CQ = dalloc<float>(cap * (size_t)L.max_cq);
         L.Q = dalloc<float>(cap * (size_t)L.max_q);
-        L.Qa = dalloc<float>(cap * (size_t)L.max_qa);
+    }
+    if (L.max_qa) L.Qa = dalloc<float>(cap * (size_t)L.max_qa);
+    if (L.max_gt) L.GT = dalloc<float>(cap * (size_t)L.max_gt);
+    if (L.ds_stride) {                 // a pass cut into more chunks than this goes token by token
+        L.ds_chunks = (int)(cap / LAY_DELTA_CHUNK) + 32;
+        L.DS = dalloc<float>((size_t)L.ds_chunks * L.ds_stride);
     }
     if (L.max_ld) L.LD = dalloc<float>(cap * (size_t)L.max_ld);
     if (L.max_mh) { L.KM = dalloc<float>(cap * (size_t)L.max_mh); L.MR = dalloc<float>(cap * (size_t)L.max_mh); }
@@ -1142,6 +1304,7 @@ void Model::alloc_runtime_layered() {
     }
     if (!L.f32) {
         int max_k = std::max({(int)W, L.max_o, L.max_ff, L.max_cq, L.max_sff}), dense_ff = L.max_sff;
+        for (const LayerSpec& sp : L.spec) max_k = std::max({max_k, sp.a_rank, sp.g_rank});
         for (const LayerSpec& sp : L.spec) if (sp.mlp == LMLP_DENSE && sp.gated_ff) dense_ff = std::max(dense_ff, sp.ff);
         const size_t rows = (cap + 255) / 256 * 256;
         L.Abf = dalloc<uint16_t>(rows * (size_t)max_k);
@@ -1183,6 +1346,7 @@ void Model::alloc_runtime_layered() {
     size_t tiles = 0;
     for (int nrep : L.nreps) tiles += 2 * (cap * (size_t)nrep / 16 + (size_t)MAXB + 1) + 2 * (cap * (size_t)nrep / LAY_ATTN_MFMA_ROWS + (size_t)MAXB + 1);
     tiles += 2 * (cap / LAY_LIGHT_CHUNK + (size_t)MAXB + 1);      // lightning chunks
+    tiles += 2 * ((size_t)L.ds_chunks + 1);                       // delta-rule chunks
     L.tab_ints = 3 * cap + (size_t)MAXB * (sizeof(LaySegDev) / 4) + (size_t)MAXB * max_pages_per_seq + tiles + 64;
     L.d_tab = dalloc<int32_t>(L.tab_ints);
     CM_HIP(hipHostMalloc((void**)&L.h_tab, L.tab_ints * sizeof(int32_t)));
@@ -1288,7 +1452,7 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
         int32_t* t_wrows = tab + o; const size_t o_wrows = o; o += (size_t)T;
         LaySegDev* t_segs = (LaySegDev*)(tab + o); const size_t o_segs = o; o += (size_t)nseg * (sizeof(LaySegDev) / 4);
         int32_t* t_bt = tab + o; const size_t o_bt = o; o += (size_t)nseg * max_pages_per_seq;
-        int nw = 0, row = 0, nchunks = 0, max_n = 0;
+        int nw = 0, row = 0, nchunks = 0, dchunks = 0, max_n = 0;
         long long max_len = 0;
         bool all_decode = true;
         for (int k = 0; k < nseg; ++k) {
@@ -1296,8 +1460,9 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
             Seq& q = seq(it.seq);
             const int n = ps[(size_t)k].n;
             const int sp = (int)q.len;
-            t_segs[k] = LaySegDev{row, n, sp, it.seq, k * max_pages_per_seq, nchunks, 0, 0};
+            t_segs[k] = LaySegDev{row, n, sp, it.seq, k * max_pages_per_seq, nchunks, dchunks, 0};
             nchunks += (n + LAY_LIGHT_CHUNK - 1) / LAY_LIGHT_CHUNK;
+            if (n > LAY_DELTA_SEQ) dchunks += (n + LAY_DELTA_CHUNK - 1) / LAY_DELTA_CHUNK;
             max_n = std::max(max_n, n);
             max_len = std::max(max_len, (long long)sp + n);
             memcpy(t_bt + (size_t)k * max_pages_per_seq, q.pages.data(), q.pages.size() * sizeof(int32_t));
@@ -1335,6 +1500,13 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
         if (L.U && max_n > LAY_LIGHT_CHUNK)
             for (int k = 0; k < nseg; ++k)
                 for (int t0 = 0; t0 < t_segs[k].n; t0 += LAY_LIGHT_CHUNK) { tab[o++] = k; tab[o++] = t0; }
+        if (o & 1) ++o;
+        const size_t o_dchunks = o;
+        if (dchunks > L.ds_chunks) dchunks = 0;
+        if (dchunks > 0)
+            for (int k = 0; k < nseg; ++k)
+                if (t_segs[k].n > LAY_DELTA_SEQ)
+                    for (int t0 = 0; t0 < t_segs[k].n; t0 += LAY_DELTA_CHUNK) { tab[o++] = k; tab[o++] = t0; }
         if (o > L.tab_ints) throw CmError(CM_ERR_INVALID, "step tables overflow");
         CM_HIP(hipMemcpyAsync(L.d_tab, tab, o * sizeof(int32_t), hipMemcpyHostToDevice, s));
         const uint32_t* d_ids = (const uint32_t*)(L.d_tab + o_ids);
@@ -1411,6 +1583,68 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
             } else
                 launch_lay_attn(a, kv_mode, s);
         };
+        // latent attention of one layer from its projection row: queries from their own latent (q_rank > 0) or straight from the row, the
+        // key latent normed into the pages (its rotated part, if any, beside it), values per head -- times the gate, if any -- into L.O2
+        auto run_latent = [&](const LayerSpec& sp, const LayeredLayerW& w) {
+            const int H = sp.heads, ev = sp.vdim, kr = sp.kv_rank, r = sp.rot_dim, dh = sp.dim, dk = kr + r;
+            const float* q = L.P + w.q_off;
+            int ldq = w.in_rows;
+            if (sp.q_rank > 0) {
+                launch_lay_rms_cols(L.P, w.in_rows, w.q_off, sp.q_rank, w.dq_norm, L.CQ, sp.q_rank, T, cfg.eps, s);
+                LGemmArgs gq;
+                gq.A = L.CQ; gq.lda = sp.q_rank; gq.W = w.uq; gq.C = L.Q; gq.ldc = H * (dh + r); gq.M = T; gq.N = H * (dh + r); gq.K = sp.q_rank;
+                lay_gemm(*this, L, gq, 1, s);
+                q = L.Q; ldq = H * (dh + r);
+            }
+            if (r > 0) {
+                launch_lay_rms_cols(L.P, w.in_rows, w.k_off, kr, w.dkv_norm, L.P + w.k_off, w.in_rows, T, cfg.eps, s);
+                if (sp.rot.dims > 0)
+                    launch_lay_rope(L.P + w.k_off + kr, w.in_rows, 0, L.P + w.k_off + kr, w.in_rows, 0, 1, r, sp.rot.dims, w.rot_freq, w.rot_mag,
+                                    d_segs, d_rowseg, T, s);
+                launch_lay_k_append(L.P, w.in_rows, w.k_off, kv_pool + w.k_pool_off, kv_mode, d_bt, d_segs, d_rowseg, T, 1, dk, page, s);
+            } else
+                launch_lay_latent_append(L.P, w.in_rows, w.k_off, kr, w.dkv_norm, cfg.eps, kv_pool + w.k_pool_off, kv_mode, d_bt, d_segs, d_rowseg, T, page, s);
+            // q_unrotated . (W_uk c) = (W_uk^T q_unrotated) . c: per head, the query moves into the latent's space
+            LGemmArgs ga;
+            ga.A = q; ga.lda = ldq; ga.a_goff = (size_t)(dh + r); ga.W = w.uk_t; ga.w_stride = (size_t)kr * dh;
+            ga.C = L.Qa; ga.ldc = H * dk; ga.c_goff = (size_t)dk; ga.M = T; ga.N = kr; ga.K = dh;
+            lay_gemm(*this, L, ga, H, s);
+            if (r > 0)
+                launch_lay_rope(q + dh, ldq, dh + r, L.Qa + kr, H * dk, dk, H, r, sp.rot.dims, w.rot_freq, w.rot_mag, d_segs, d_rowseg, T, s);
+            run_attention(sp, w, L.Qa, H * dk, 0, 0, dk, kr);
+            // the weighted latents become values per head, times the gate
+            LGemmArgs gv;
+            gv.A = L.O; gv.lda = H * kr; gv.a_goff = (size_t)kr; gv.W = w.uv; gv.w_stride = (size_t)ev * kr;
+            gv.C = L.O2; gv.ldc = H * ev; gv.c_goff = (size_t)ev; gv.M = T; gv.N = ev; gv.K = kr;
+            if (sp.gate_latent) { gv.mul = L.P + w.g_off; gv.ldm = w.in_rows; }
+            lay_gemm(*this, L, gv, H, s);
+        };
+        // gated delta rule of one layer: gated head outputs into L.O2
+        auto run_delta = [&](const LayerSpec& sp, const LayeredLayerW& w) {
+            const int H = sp.heads, d = sp.dim, e = sp.vdim;
+            LDeltaArgs a;
+            a.proj = L.P; a.ldp = w.in_rows; a.q_off = w.q_off; a.b_off = w.b_off; a.a_off = w.a_off;
+            a.H = H; a.G = sp.kv_heads; a.d = d; a.e = e;
+            a.conv_w = w.conv_w; a.taps = sp.conv; a.conv_pool = conv_pool; a.conv_stride = conv_slot_elems; a.cv_off = w.cv_off;
+            a.dt_bias = w.dt_bias; a.a_neg = w.a_neg; a.xb = L.XB; a.beta = L.KM; a.ldec = L.LD; a.channel = sp.channel_decay;
+            a.state_pool = state_pool; a.slot_stride = state_slot_elems; a.st_off = w.st_off;
+            a.segs = d_segs; a.rowseg = d_rowseg; a.nseg = nseg; a.T = T;
+            a.gate = L.P + w.g_off; a.ldg = w.in_rows; a.norm_w = w.mix_norm; a.eps = cfg.eps;
+            a.o_raw = L.O; a.out = L.O2; a.all_single = all_decode;
+            if (dchunks > 0) { a.chunks = (const int2*)(L.d_tab + o_dchunks); a.nchunks = dchunks; a.scratch = L.DS; }
+            if (sp.channel_decay) {            // softplus of the decay's low-rank pair, sigmoid of the gate's
+                LGemmArgs gd;
+                gd.A = L.P + w.a_off; gd.lda = w.in_rows; gd.W = w.a2; gd.bias = w.dt_bias; gd.C = L.LD; gd.ldc = H * d; gd.M = T; gd.N = H * d; gd.K = sp.a_rank;
+                gd.act = LACT_SOFTPLUS; gd.act_split = gd.N;
+                lay_gemm(*this, L, gd, 1, s);
+                LGemmArgs gg;
+                gg.A = L.P + w.g_off; gg.lda = w.in_rows; gg.W = w.g2; gg.C = L.GT; gg.ldc = H * e; gg.M = T; gg.N = H * e; gg.K = sp.g_rank;
+                gg.act = LACT_SIGMOID; gg.act_split = gg.N;
+                lay_gemm(*this, L, gg, 1, s);
+                a.gate = L.GT; a.ldg = H * e;
+            }
+            launch_lay_delta(a, s);
+        };
         // lightning / gated linear attention of one layer: raw head outputs into L.O
         // ldp: width of the projection rows in L.P; kmul != null: the matrix-memory form (one decay and one key factor per head and
         // token, a constant 1 as last value column, raw outputs [T][H (e + 1)] into L.O2)
@@ -1439,10 +1673,10 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
             }
         };
         // pre-norm layers: the finished sublayer's rows (nsum per token, summed in order) join the residual inside the next norm's launch
-        struct { const float* y = nullptr; int nsum = 1; } padd;
+        struct { const float* y = nullptr; int nsum = 1; const float* wsel = nullptr; } padd;
         auto add_gnorm = [&](const float* nw_, float* out) {
-            launch_lay_add_gnorm(L.X, nullptr, padd.y, padd.nsum, nw_, out, T, W, L.norm_groups, cfg.eps, s);
-            padd.y = nullptr;
+            launch_lay_add_gnorm(L.X, nullptr, padd.y, padd.nsum, nw_, out, T, W, L.norm_groups, cfg.eps, s, padd.wsel);
+            padd.y = nullptr; padd.wsel = nullptr;
         };
         const float *par_y1 = nullptr, *par_y2 = nullptr;       // parallel layers: sublayer outputs not yet added to the residual
         for (size_t li = 0; li < L.spec.size(); ++li) {
@@ -1473,32 +1707,7 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
                     }
                     run_attention(sp, w, L.P, w.in_rows, w.q_off, w.g_off, sp.dim, ev);
                 } else if (sp.mixer == LMIX_LATENT) {
-                    const int kr = sp.kv_rank, r = sp.rot_dim, dh = sp.dim, dk = kr + r;
-                    // both latents through their norms; the key latent in place, next to the shared rotated key part
-                    launch_lay_rms_cols(L.P, w.in_rows, w.q_off, sp.q_rank, w.dq_norm, L.CQ, sp.q_rank, T, cfg.eps, s);
-                    launch_lay_rms_cols(L.P, w.in_rows, w.k_off, kr, w.dkv_norm, L.P + w.k_off, w.in_rows, T, cfg.eps, s);
-                    LGemmArgs gq;
-                    gq.A = L.CQ; gq.lda = sp.q_rank; gq.W = w.uq; gq.C = L.Q; gq.ldc = H * (dh + r); gq.M = T; gq.N = H * (dh + r); gq.K = sp.q_rank;
-                    lay_gemm(*this, L, gq, 1, s);
-                    if (r > 0 && sp.rot.dims > 0)
-                        launch_lay_rope(L.P + w.k_off + kr, w.in_rows, 0, L.P + w.k_off + kr, w.in_rows, 0, 1, r, sp.rot.dims, w.rot_freq, w.rot_mag,
-                                        d_segs, d_rowseg, T, s);
-                    launch_lay_k_append(L.P, w.in_rows, w.k_off, kv_pool + w.k_pool_off, kv_mode, d_bt, d_segs, d_rowseg, T, 1, dk, page, s);
-                    // q_unrotated . (W_uk c) = (W_uk^T q_unrotated) . c: per head, the query moves into the latent's space
-                    LGemmArgs ga;
-                    ga.A = L.Q; ga.lda = H * (dh + r); ga.a_goff = (size_t)(dh + r); ga.W = w.uk_t; ga.w_stride = (size_t)kr * dh;
-                    ga.C = L.Qa; ga.ldc = H * dk; ga.c_goff = (size_t)dk; ga.M = T; ga.N = kr; ga.K = dh;
-                    lay_gemm(*this, L, ga, H, s);
-                    if (r > 0)
-                        launch_lay_rope(L.Q + dh, H * (dh + r), dh + r, L.Qa + kr, H * dk, dk, H, r, sp.rot.dims, w.rot_freq, w.rot_mag, d_segs,
-                                        d_rowseg, T, s);
-                    run_attention(sp, w, L.Qa, H * dk, 0, 0, dk, kr);
-                    // the weighted latents become values per head, times the gate
-                    LGemmArgs gv;
-                    gv.A = L.O; gv.lda = H * kr; gv.a_goff = (size_t)kr; gv.W = w.uv; gv.w_stride = (size_t)ev * kr;
-                    gv.C = L.O2; gv.ldc = H * ev; gv.c_goff = (size_t)ev; gv.M = T; gv.N = ev; gv.K = kr;
-                    gv.mul = L.P + w.g_off; gv.ldm = w.in_rows;
-                    lay_gemm(*this, L, gv, H, s);
+                    run_latent(sp, w);
                     oa = L.O2;
                 } else {
                     // logarithm of the decay: ln(sigmoid(z)^(1 / tau)), z from the low-rank pair
@@ -1532,7 +1741,8 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
                 add_gnorm(w.norm1, L.Hc);
                 LGemmArgs g;
                 g.A = L.Hc; g.lda = W; g.W = w.in_w; g.bias = w.in_b; g.C = L.P; g.ldc = w.in_rows; g.M = T; g.N = w.in_rows; g.K = W;
-                g.act_split = w.g_off; g.act = sp.mixer == LMIX_HGRN ? LACT_SILU : LACT_NONE; g.act2 = LACT_NONE;
+                g.act_split = w.g_off; g.act = sp.mixer == LMIX_HGRN ? LACT_SILU : LACT_NONE;
+                g.act2 = sp.mixer == LMIX_DELTA && !sp.channel_decay ? LACT_SILU : LACT_NONE;
                 lay_gemm(*this, L, g, 1, s);
                 const float* oa = L.O;
                 int on = 0;
@@ -1574,6 +1784,10 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
                     launch_lay_lightning(a, s);
                     launch_lay_rms_gate(L.O, nullptr, 0, w.mix_norm, L.O2, T, H * e, cfg.eps, s, e, true);
                     oa = L.O2; on = H * e;
+                } else if (sp.mixer == LMIX_LATENT || sp.mixer == LMIX_DELTA) {
+                    if (sp.mixer == LMIX_LATENT) run_latent(sp, w);
+                    else run_delta(sp, w);
+                    oa = L.O2; on = sp.heads * sp.vdim;
                 } else {
                     for (const LayerSpec& sd : sp.side) on += sd.heads * sd.vdim;
                     for (size_t k = 0; k < sp.side.size(); ++k) {
@@ -1632,9 +1846,20 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
                 go.A = oa; go.lda = on; go.W = w.o_w; go.C = L.Y; go.ldc = W; go.M = T; go.N = W; go.K = on;
                 lay_gemm(*this, L, go, 1, s);
                 padd.y = L.Y; padd.nsum = 1;
-                if (sp.mlp == LMLP_MOE) {
+                if (sp.mlp == LMLP_DENSE) {
                     add_gnorm(w.norm2, L.Hc);
-                    // an expert's weight multiplies its INPUT: the rows of the grouped product are w h, and the combine is a plain sum
+                    LGemmArgs gu;
+                    gu.A = L.Hc; gu.lda = W; gu.W = w.gate; gu.W2 = w.up; gu.C = L.HH; gu.ldc = sp.ff; gu.M = T; gu.N = sp.ff; gu.K = W;
+                    gu.act = sp.ff_act; gu.act_param = sp.limit;
+                    lay_gemm(*this, L, gu, 1, s);
+                    LGemmArgs dn;
+                    dn.A = L.HH; dn.lda = sp.ff; dn.W = w.down; dn.C = L.Y; dn.ldc = W; dn.M = T; dn.N = W; dn.K = sp.ff;
+                    lay_gemm(*this, L, dn, 1, s);
+                    padd.y = L.Y; padd.nsum = 1;
+                } else if (sp.mlp == LMLP_MOE) {
+                    add_gnorm(w.norm2, L.Hc);
+                    // scale_input: an expert's weight multiplies its INPUT, the rows of the grouped product are w h and the combine is a plain
+                    // sum; otherwise the weights join in the combine
                     const int slots = sp.top + (sp.shared_ff > 0 ? 1 : 0);
                     launch_lay_router(L.Hc, w.router, L.sel, L.wsel, T, W, sp.experts, sp.top, s, &sp.router, nullptr, slots, L.Z);
                     launch_lay_moe_plan(L.sel, L.off, L.srt, T * sp.top, sp.experts, s, sp.top, slots);
@@ -1657,7 +1882,7 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
                         sdn.N = W; sdn.K = sp.shared_ff;
                         lay_gemm(*this, L, sdn, 1, s);
                     }
-                    padd.y = L.YS; padd.nsum = slots;
+                    padd.y = L.YS; padd.nsum = slots; padd.wsel = sp.scale_input ? nullptr : L.wsel;
                 }
                 if (L.capture || li + 1 == L.spec.size()) add_gnorm(nullptr, nullptr);
             } else if (L.post_only) {
@@ -1813,6 +2038,7 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
             else launch_lay_rms_rows(L.X, d_wrows + w0, L.final_norm, L.Xw, nr, W, cfg.eps, s);
             LGemmArgs hd;
             hd.A = L.Xw; hd.lda = W; hd.W = L.head; hd.C = logitsb; hd.ldc = V; hd.M = nr; hd.N = V; hd.K = W;
+            if (L.logit_cap > 0.f) { hd.act = LACT_SOFTCAP; hd.act_split = V; hd.act_param = L.logit_cap; }
             lay_gemm(*this, L, hd, 1, s);
             if (greedy_out) {
                 launch_lay_argmax_rows(logitsb, V, V, L.d_greedy, nr, L.am_pv, L.am_pi, s);
@@ -1855,7 +2081,7 @@ uint64_t Model::layered_decode_bytes(size_t ctx) const {
             uint64_t row = (uint64_t)sp.kv_heads * sp.dim + (sp.own_v ? (uint64_t)sp.kv_heads * sp.vdim : 0);      // cached elements per token
             if (sp.mixer == LMIX_LATENT) {
                 row = (uint64_t)sp.kv_rank + sp.rot_dim;
-                n += 2ull * (H * (sp.dim + sp.rot_dim) * sp.q_rank + H * sp.dim * sp.kv_rank + H * sp.vdim * sp.kv_rank);
+                n += 2ull * (H * (sp.dim + sp.rot_dim) * sp.q_rank + H * sp.dim * sp.kv_rank + H * sp.vdim * sp.kv_rank);      // (no query latent: q_rank 0)
             }
             n += 2ull * W * H * sp.vdim;
             uint64_t seen = std::min<uint64_t>(ctx, (uint64_t)std::min<long long>(sp.win, 1ll << 40) + (uint64_t)sp.keep);
@@ -1866,7 +2092,7 @@ uint64_t Model::layered_decode_bytes(size_t ctx) const {
             n += 2ull * W * sp.heads * sp.vdim + 8ull * sp.heads * sp.dim * (sp.vdim + 1);
         } else {
             n += 2ull * W * sp.heads * sp.vdim + 8ull * sp.heads * sp.dim * sp.vdim;    // state read + write
-            if (sp.mixer == LMIX_GLA) n += 2ull * sp.heads * sp.dim * sp.a_rank;
+            if (sp.mixer == LMIX_GLA || sp.mixer == LMIX_DELTA) n += 2ull * sp.heads * (sp.dim * sp.a_rank + sp.vdim * sp.g_rank);
         }
         return n;
     };
