@@ -318,6 +318,43 @@ CONFIGS.update({
 })
 
 
+# ---- layer-list decoders: Rirotar ------------------------------------------------------------------------------------------
+def rirotar_config(vocab: int, width: int, kinds: "list | tuple", ff: int, lat_heads: int, lat_dim: int, lat_vdim: int, kv_rank: int,
+                   window: int, del_heads: int, del_kv_heads: int, del_dim: int, del_vdim: int, experts: int, top: int, expert_ff: int,
+                   groups: int = 1, keep_groups: int = 1, router_scale: float = 2.5, conv: int = 4, limit: float = 7.0, softcap: float = 30.0,
+                   eps: float = 1e-6, routed: "tuple | list" = (), no_ff: "tuple | list" = ()) -> dict:
+    """Layers of the kinds named in `kinds`: "latent_attention" (one cached latent per token, sliding window, sinks), "delta" (gated
+    delta rule, a decay per head) and "channel_delta" (a decay per key channel); dense feed-forwards, mixtures of experts in the layers
+    of `routed`, none in those of `no_ff`."""
+    layers = []
+    for i, kind in enumerate(kinds):
+        if kind == "latent_attention":
+            mx = dict(heads=lat_heads, dim=lat_dim, vdim=lat_vdim, kv_rank=kv_rank, scale=lat_dim ** -0.5, mask=dict(size=window))
+        else:
+            mx = dict(heads=del_heads, kv_heads=del_kv_heads if kind == "delta" else del_heads, dim=del_dim, vdim=del_vdim, conv=conv)
+        mlp = dict(kind="dense", ff=ff, limit=limit)
+        if i in routed:
+            mlp = dict(kind="moe", expert=dict(ff=expert_ff, limit=limit),
+                       router=dict(experts=experts, top=top, groups=dict(count=groups, keep=keep_groups), scale=router_scale))
+        layers.append(dict(type=kind, mixer=mx, mlp=None if i in no_ff else mlp))
+    return dict(architecture="Rirotar", vocab=vocab, width=width, norm=dict(eps=eps), logit_softcap=softcap, layers=layers)
+
+
+_RIROTAR_1B = dict(ff=3584, lat_heads=8, lat_dim=128, lat_vdim=128, kv_rank=512, window=1024, del_heads=16, del_kv_heads=8, del_dim=128,
+                   del_vdim=128, experts=16, top=4, expert_ff=896, groups=4, keep_groups=2)
+CONFIGS.update({
+    "tiny-rirotar": rirotar_config(320, 128, ["delta", "latent_attention", "channel_delta", "delta", "latent_attention"], ff=192, lat_heads=2,
+                                   lat_dim=16, lat_vdim=24, kv_rank=32, window=20, del_heads=4, del_kv_heads=2, del_dim=16, del_vdim=24,
+                                   experts=6, top=2, expert_ff=48, groups=3, keep_groups=2, conv=3, limit=1.5, softcap=12.0, routed=(1, 3),
+                                   no_ff=(2,)),
+    # the widths of the Qwen3.5-0.8B text decoder, mononex-1b and korupel-1b-moe (1024 wide, 3584 ff, 24 layers, vocabulary 248 320): 12 delta
+    # rules with a decay per head and 6 with a decay per key channel (16 heads of 128 x 128), 6 latent attention layers (8 heads of 128, latent
+    # 512, window 1024); every second feed-forward is a mixture of 16 experts of 896 in 4 groups, 4 per token
+    "rirotar-1b": rirotar_config(248320, 1024, ["delta", "channel_delta", "delta", "latent_attention"] * 6, routed=tuple(range(1, 24, 2)), **_RIROTAR_1B),
+    "rirotar-1b-4l": rirotar_config(32768, 1024, ["delta", "channel_delta", "delta", "latent_attention"], routed=(1, 3), **_RIROTAR_1B),
+})
+
+
 def get_config(name: str) -> dict:
     if name not in CONFIGS:
         raise KeyError(f"unknown config {name!r}; have {sorted(CONFIGS)}")

@@ -312,30 +312,33 @@ __global__ __launch_bounds__(256) void lay_delta_out_kernel(LDeltaArgs a, int ma
 // chunk_prep (chunk, head, value slice): M, B, R, Y0;  chunk_scan (sequence, head, 16 value columns): the states S0 of all chunks, the only
 // sequential part, one product per chunk;  chunk_out (chunk, head): O with the head norm and the output gate.
 // Every exponent is a difference <= 0: tiles of A and P off the diagonal take the last position in front of the row tile as reference
-// (e^(b_t - ref) e^(ref - b_s)), tiles on it form each pair's own.
+// (e^(b_t - ref) e^(ref - b_s)), tiles on it form each pair's own.  So that strong decays earlier in a chunk do not cost the later small
+// differences their digits, the head form keeps b in 64 bits; the channel form keeps the sums of each tile of 16 tokens by themselves and
+// stops ln g at LN_FLOOR, where everything older is far below the rounding of what is written next.
 // Scratch per (chunk, head), DP = 64 or 128 >= d, EP = e rounded up to 16: M [DP][DP] | B, then S0, transposed [EP][DP] | R [64][DP] | Y0 [64][EP]
 // ------------------------------------------------------------------------------------------------------------------
 constexpr int DC = LAY_DELTA_CHUNK, DCP = DC + 4, DV = 128;
+constexpr float LN_FLOOR = -30.f;
 static int ld_dp(int d) { return d <= 64 ? 64 : 128; }
 __host__ __device__ static inline int ld_ep(int e) { return (e + 15) / 16 * 16; }
 __host__ __device__ static inline size_t ld_floats(int dp, int e) { return (size_t)dp * dp + (size_t)ld_ep(e) * dp + (size_t)DC * dp + (size_t)DC * ld_ep(e); }
 bool lay_delta_chunk_fits(int d, int e) { return d > 0 && e > 0 && d <= 128 && e <= 256; }
 size_t lay_delta_chunk_floats(int d, int e) { return ld_floats(ld_dp(d), e); }
 
-static size_t lay_delta_prep_lds(int DP) { return (size_t)(3 * DC * (DP + 4) + 2 * DC * DCP + 4 * 16 * 20 + 2 * DC + DP) * sizeof(float); }
+static size_t lay_delta_prep_lds(int DP) { return (size_t)(3 * DC * (DP + 4) + 2 * DC * DCP + 4 * 16 * 20 + 3 * DC + 4 * DP) * sizeof(float); }
 template <bool CH, int DP>
 __global__ __launch_bounds__(512) void lay_delta_chunk_prep_kernel(LDeltaArgs a) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
     constexpr int KP = DP + 4, ND = DP / 16;
     float (*Ks)[KP] = (float (*)[KP])sm;                       // K, then beta e^b K
     float (*Qs)[KP] = (float (*)[KP])(sm + DC * KP);           // Q, then e^b Q
-    float (*Bs)[KP] = (float (*)[KP])(sm + 2 * DC * KP);       // channel form: b; then Kd
+    float (*Bs)[KP] = (float (*)[KP])(sm + 2 * DC * KP);       // channel form: b from the start of the token's tile; then Kd
     float (*Am)[DCP] = (float (*)[DCP])(sm + 3 * DC * KP);     // -A
     float (*Pm)[DCP] = (float (*)[DCP])(sm + 3 * DC * KP + DC * DCP);
     float (*Ti)[16][20] = (float (*)[16][20])(sm + 3 * DC * KP + 2 * DC * DCP);      // inverses of the diagonal tiles of I + A
-    float* lg = sm + 3 * DC * KP + 2 * DC * DCP + 4 * 16 * 20; // head form: b
-    float* bt = lg + DC;                                       // beta
-    float* bc = bt + DC;                                       // [DP] b at the chunk's last token
+    double* lg = (double*)(sm + 3 * DC * KP + 2 * DC * DCP + 4 * 16 * 20);           // head form: b
+    float* bt = (float*)(lg + DC);                             // beta
+    float (*tot)[DP] = (float (*)[DP])(bt + DC);               // channel form: the tiles' sums
     const int2 chk = a.chunks[blockIdx.x];
     const LaySegDev sg = a.segs[chk.x];
     const int n = min(DC, sg.n - chk.y), row0 = sg.row0 + chk.y;
@@ -349,34 +352,26 @@ __global__ __launch_bounds__(512) void lay_delta_chunk_prep_kernel(LDeltaArgs a)
         const float* x = a.xb + (size_t)(row0 + (in ? t : 0)) * C + kh * d + (in ? i : 0);
         Qs[t][i] = in ? x[0] : 0.f;
         Ks[t][i] = in ? x[a.G * d] : 0.f;
-        if (CH) Bs[t][i] = in ? an * a.ldec[((size_t)(row0 + t) * a.H + h) * d + i] : 0.f;
+        if (CH) Bs[t][i] = in ? fmaxf(an * a.ldec[((size_t)(row0 + t) * a.H + h) * d + i], LN_FLOOR) : 0.f;
     }
     for (int idx = tid; idx < 2 * DC * DCP; idx += 512) (&Am[0][0])[idx] = 0.f;
     if (wave == 0) {
         bt[lane] = lane < n ? a.beta[(size_t)(row0 + lane) * a.H + h] : 0.f;
         if (!CH) {
-            float g = lane < n ? a.ldec[(size_t)(row0 + lane) * a.H + h] : 0.f;
+            double g = lane < n ? (double)a.ldec[(size_t)(row0 + lane) * a.H + h] : 0.0;
 #pragma unroll
-            for (int s = 1; s < 64; s <<= 1) { const float o = __shfl_up(g, s); if (lane >= s) g += o; }
+            for (int s = 1; s < 64; s <<= 1) { const double o = __shfl_up(g, s); if (lane >= s) g += o; }
             lg[lane] = g;
         }
     }
     __syncthreads();
-    if (CH) {                              // running sums down the tokens: 16 rows per thread, then the rows in front
+    if (CH) {                              // running sums down the tokens of each tile
         const int i = tid % DP, q4 = tid / DP;
         if (q4 < 4) {
             float run = 0.f;
 #pragma unroll
             for (int t = 0; t < 16; ++t) { run += Bs[16 * q4 + t][i]; Bs[16 * q4 + t][i] = run; }
-        }
-        __syncthreads();
-        float off = 0.f;
-        if (q4 < 4) for (int p = 0; p < q4; ++p) off += Bs[16 * p + 15][i];
-        __syncthreads();
-        if (q4 < 4) {
-#pragma unroll
-            for (int t = 0; t < 16; ++t) Bs[16 * q4 + t][i] += off;
-            if (q4 == 3) bc[i] = Bs[63][i];
+            tot[q4][i] = run;
         }
         __syncthreads();
     }
@@ -394,17 +389,18 @@ __global__ __launch_bounds__(512) void lay_delta_chunk_prep_kernel(LDeltaArgs a)
             f32x4 av = *(const f32x4*)&(which ? Qs : Ks)[16 * tr + r][16 * jj + 4 * kq];
             f32x4 bv = *(const f32x4*)&Ks[16 * tc + r][16 * jj + 4 * kq];
             if (CH) {
-                const f32x4 ref = *(const f32x4*)&Bs[16 * tr - 1][16 * jj + 4 * kq];
-                const f32x4 ba = *(const f32x4*)&Bs[16 * tr + r][16 * jj + 4 * kq], bb = *(const f32x4*)&Bs[16 * tc + r][16 * jj + 4 * kq];
+                const f32x4 ba = *(const f32x4*)&Bs[16 * tr + r][16 * jj + 4 * kq];
+                f32x4 bb = *(const f32x4*)&tot[tc][16 * jj + 4 * kq] - *(const f32x4*)&Bs[16 * tc + r][16 * jj + 4 * kq];
+                for (int m = tc + 1; m < tr; ++m) bb += *(const f32x4*)&tot[m][16 * jj + 4 * kq];
 #pragma unroll
-                for (int i = 0; i < 4; ++i) { av[i] *= __expf(ba[i] - ref[i]); bv[i] *= __expf(ref[i] - bb[i]); }
+                for (int i = 0; i < 4; ++i) { av[i] *= __expf(ba[i]); bv[i] *= __expf(bb[i]); }
             }
             acc = dl_mfma(av, bv, acc);
         }
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int t = 16 * tr + 4 * kq + i, s = 16 * tc + r;
-            const float f = CH ? 1.f : (s <= t ? expf(lg[t] - lg[s]) : 0.f);
+            const float f = CH ? 1.f : (s <= t ? expf((float)(lg[t] - lg[s])) : 0.f);
             if (which) Pm[t][s] = f * acc[i];
             else Am[t][s] = s < t ? -bt[t] * f * acc[i] : 0.f;
         }
@@ -441,8 +437,15 @@ __global__ __launch_bounds__(512) void lay_delta_chunk_prep_kernel(LDeltaArgs a)
     // ---- K, Q -> beta e^b K, e^b Q, Kd (a thread touches its own elements only); inverses of the diagonal tiles by the last wave
     for (int idx = tid; idx < DC * DP; idx += 512) {
         const int t = idx / DP, i = idx % DP;
-        const float b = CH ? Bs[t][i] : lg[t], end = CH ? bc[i] : lg[DC - 1], eb = expf(b), k = Ks[t][i];
-        Bs[t][i] = k * expf(end - b);
+        const float k = Ks[t][i];
+        float b, rest;                     // ln of the decay from the chunk's start to token t, and from there to its end
+        if (CH) {
+            b = Bs[t][i]; rest = tot[t >> 4][i] - b;
+            for (int m = 0; m < t >> 4; ++m) b += tot[m][i];
+            for (int m = (t >> 4) + 1; m < 4; ++m) rest += tot[m][i];
+        } else { b = (float)lg[t]; rest = (float)(lg[DC - 1] - lg[t]); }
+        const float eb = expf(b);
+        Bs[t][i] = k * expf(rest);
         Ks[t][i] = bt[t] * k * eb;
         Qs[t][i] *= eb;
     }
@@ -518,7 +521,7 @@ __global__ __launch_bounds__(512) void lay_delta_chunk_prep_kernel(LDeltaArgs a)
             f32x4 acc = {0.f, 0.f, 0.f, 0.f};
             if (isw) {
 #pragma unroll
-                for (int i = 0; i < 4; ++i) if (16 * m + 4 * kq + i == c) acc[i] = expf(CH ? bc[c] : lg[DC - 1]);
+                for (int i = 0; i < 4; ++i) if (16 * m + 4 * kq + i == c) acc[i] = expf(CH ? (tot[0][c] + tot[1][c]) + (tot[2][c] + tot[3][c]) : (float)lg[DC - 1]);
             }
 #pragma unroll
             for (int L = 0; L < 4; ++L) {
