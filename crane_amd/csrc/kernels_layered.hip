@@ -15,7 +15,6 @@ __device__ __forceinline__ float lay_act(float v, int act, float param = 1.f) {
     switch (act) {
         case LACT_RELU2: { const float r = fmaxf(v, 0.f); return r * r; }
         case LACT_LOGSIG: return param * (fminf(v, 0.f) - log1pf(expf(-fabsf(v))));      // ln sigmoid(v), no overflow either way
-        case LACT_SOFTPLUS: return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v)));
         case LACT_SOFTCAP: return param * tanhf(v / param);
         case LACT_SILU: return v / (1.f + __expf(-v));
         case LACT_SIGMOID: return 1.f / (1.f + __expf(-v));

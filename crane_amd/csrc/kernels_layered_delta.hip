@@ -23,6 +23,9 @@ __device__ __forceinline__ float dl_silu(float v) { return v / (1.f + expf(-v));
 __device__ __forceinline__ float dl_sigmoid(float v) { return 1.f / (1.f + expf(-v)); }
 __device__ __forceinline__ float dl_softplus(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
 
+// output gates (not part of the recurrence): the hardware exponential
+__device__ __forceinline__ float dl_gate(float v, int act) { return (act == LACT_SILU ? v : 1.f) / (1.f + __expf(-v)); }
+
 // workgroup barrier for LDS hand-offs: waits for this wave's LDS operations, not for its outstanding global loads
 __device__ __forceinline__ void dl_lds_barrier() {
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -41,35 +44,44 @@ __device__ __forceinline__ f32x4 dl_mfma(const f32x4& a, const f32x4& b, f32x4 c
 }  // namespace
 
 // ------------------------------------------------------------------------------------------------------------------
-// latent row: norm and cache append, one wave per row
+// latent row: norm and cache append, one block per row
 // ------------------------------------------------------------------------------------------------------------------
 template <int KVT>
 __global__ __launch_bounds__(256) void lay_latent_append_kernel(const float* __restrict__ proj, int ldp, int k_off, int n, const float* __restrict__ w,
                                                                 float eps, void* __restrict__ kpool, const int32_t* __restrict__ bt,
-                                                                const LaySegDev* __restrict__ segs, const int32_t* __restrict__ rowseg, int T,
-                                                                int page) {
-    const int r = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (r >= T) return;
+                                                                const LaySegDev* __restrict__ segs, const int32_t* __restrict__ rowseg, int page) {
+    __shared__ float red[4];
+    const int r = blockIdx.x, tid = threadIdx.x;
+    const float* x = proj + (size_t)r * ldp + k_off;
+    float v[2], ss = 0.f;                  // the thread's first two elements stay in registers (the whole row up to a latent of 512)
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int c = tid + 256 * i;
+        v[i] = c < n ? x[c] : 0.f;
+        ss = fmaf(v[i], v[i], ss);
+    }
+    for (int c = tid + 512; c < n; c += 256) ss = fmaf(x[c], x[c], ss);
     const LaySegDev sg = segs[rowseg[r]];
     const int pos = sg.start_pos + (r - sg.row0);
-    const float* x = proj + (size_t)r * ldp + k_off;
-    float ss = 0.f;
-    for (int c = lane; c < n; c += 64) { const float v = x[c]; ss += v * v; }
-    ss = wave_sum(ss);
-    const float rs = 1.f / sqrtf(ss / (float)n + eps);
     const size_t row = ((size_t)bt[sg.bt_off + pos / page] * page + (size_t)(pos % page)) * n;
-    for (int c = lane; c < n; c += 64) {
-        const float v = x[c] * rs * w[c];
-        if (KVT == KV_F32) ((float*)kpool)[row + c] = v;
-        else ((uint16_t*)kpool)[row + c] = f32_to_bf16(v);
-    }
+    ss = wave_sum(ss);
+    if ((tid & 63) == 0) red[tid >> 6] = ss;
+    __syncthreads();
+    const float rs = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)n + eps);
+    auto put = [&](int c, float y) {
+        if (KVT == KV_F32) ((float*)kpool)[row + c] = y;
+        else ((uint16_t*)kpool)[row + c] = f32_to_bf16(y);
+    };
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+        if (tid + 256 * i < n) put(tid + 256 * i, v[i] * rs * w[tid + 256 * i]);
+    for (int c = tid + 512; c < n; c += 256) put(c, x[c] * rs * w[c]);
 }
 void launch_lay_latent_append(const float* proj, int ldp, int k_off, int n, const float* w, float eps, void* kpool, int kvt, const int32_t* bt,
                               const LaySegDev* segs, const int32_t* rowseg, int T, int page, hipStream_t s) {
-    if (T <= 0) return;
-    const dim3 grid((unsigned)((T + 3) / 4));
-    if (kvt == KV_F32) hipLaunchKernelGGL(lay_latent_append_kernel<KV_F32>, grid, dim3(256), 0, s, proj, ldp, k_off, n, w, eps, kpool, bt, segs, rowseg, T, page);
-    else hipLaunchKernelGGL(lay_latent_append_kernel<KV_BF16>, grid, dim3(256), 0, s, proj, ldp, k_off, n, w, eps, kpool, bt, segs, rowseg, T, page);
+    if (T <= 0 || n <= 0) return;
+    if (kvt == KV_F32) hipLaunchKernelGGL(lay_latent_append_kernel<KV_F32>, dim3((unsigned)T), dim3(256), 0, s, proj, ldp, k_off, n, w, eps, kpool, bt, segs, rowseg, page);
+    else hipLaunchKernelGGL(lay_latent_append_kernel<KV_BF16>, dim3((unsigned)T), dim3(256), 0, s, proj, ldp, k_off, n, w, eps, kpool, bt, segs, rowseg, page);
 }
 
 // ------------------------------------------------------------------------------------------------------------------
@@ -169,22 +181,17 @@ __global__ __launch_bounds__(256) void lay_delta_prep_kernel(LDeltaArgs a) {
 // FUSED (decode steps): the block forms its own q, k, v, write strength and decay; only lay_delta_out replaces the convolution's tail.
 // ------------------------------------------------------------------------------------------------------------------
 constexpr int LQ_COLS = 32, LQ_GRP = 8;
+constexpr int lq_batch(bool fused, int nr) { return fused ? 1 : (nr > 16 ? 8 : 16); }      // tokens staged at once
 template <bool FUSED, int NR>
 __global__ __launch_bounds__(256) void lay_delta_seq_kernel(LDeltaArgs a, int max_n) {
-    extern __shared__ float lds[];
-    constexpr int TB = FUSED ? 1 : LAY_DELTA_SEQ;
+    constexpr int TB = lq_batch(FUSED, NR), ROWS = NR * LQ_GRP;
+    __shared__ __attribute__((aligned(16))) f32x4 qkg[TB][ROWS];       // {q, k, g, -} per key row; rows past d are zero
+    __shared__ float vs[TB][LQ_COLS], bs[TB], part[2][LQ_GRP][LQ_COLS][2], kqs[2][LQ_GRP], red[4];
     const LaySegDev sg = a.segs[blockIdx.x];
     if (sg.n > max_n) return;              // the chunk-parallel form takes this portion
     const int d = a.d, e = a.e, h = blockIdx.y, kh = h / (a.H / a.G), j0 = blockIdx.z * LQ_COLS;
     const int C = 2 * a.G * d + a.H * e;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, j = tid & (LQ_COLS - 1), rg = tid / LQ_COLS;
-    float* qs = lds;                       // [TB][d]
-    float* ks = qs + TB * d;               // [TB][d]
-    float* gs = ks + TB * d;               // [TB][d] decays
-    float* vs = gs + TB * d;               // [TB][32]
-    float* bs = vs + TB * LQ_COLS;         // [TB]
-    float* part = bs + TB;                 // [2][8][32][2]
-    float* red = part + 2 * LQ_GRP * LQ_COLS * 2;      // [4]
     const int col = j0 + j;
     const bool ok = col < e;
     float* st = a.state_pool + (size_t)sg.slot * a.slot_stride + a.st_off + (size_t)h * d * e + min(col, e - 1);
@@ -196,75 +203,86 @@ __global__ __launch_bounds__(256) void lay_delta_seq_kernel(LDeltaArgs a, int ma
         const int nt = min(TB, sg.n - t0);
         if (!FUSED) __syncthreads();       // the previous batch is consumed
         if (FUSED) {
-            // the head's query and key channels: two waves each
+            // the head's query (waves 0, 1) and key channels (waves 2, 3), a thread's channels in registers until their length is known
             const float* tail = a.conv_pool + (size_t)sg.slot * a.conv_stride + a.cv_off;
             const float* x = a.proj + (size_t)sg.row0 * a.ldp + a.q_off;
             auto conv = [&](int c) {
                 float acc = 0.f;
-                for (int k = 0; k + 1 < a.taps; ++k) acc = fmaf(a.conv_w[(size_t)c * a.taps + k], tail[(size_t)k * C + c], acc);
-                return dl_silu(fmaf(a.conv_w[(size_t)c * a.taps + a.taps - 1], x[c], acc));
+                for (int k0 = 0; k0 < a.taps; k0 += 4) {             // four taps' loads in flight
+                    float w[4], v[4];
+#pragma unroll
+                    for (int k = 0; k < 4; ++k) {
+                        const int kk = min(k0 + k, a.taps - 1);
+                        w[k] = a.conv_w[(size_t)c * a.taps + kk];
+                        const float* p = kk < a.taps - 1 ? tail + (size_t)kk * C : x;
+                        v[k] = p[c];
+                    }
+#pragma unroll
+                    for (int k = 0; k < 4; ++k) if (k0 + k < a.taps) acc = fmaf(w[k], v[k], acc);
+                }
+                return dl_silu(acc);
             };
-            float ss = 0.f;
-            for (int i = (wave & 1) * 64 + lane; i < d; i += 128) {
-                const float y = conv((wave < 2 ? 0 : a.G * d) + kh * d + i);
-                (wave < 2 ? qs : ks)[i] = y;
-                ss = fmaf(y, y, ss);
+            constexpr int PT = (ROWS + 127) / 128;
+            const int i0 = (wave & 1) * 64 + lane, base = (wave < 2 ? 0 : a.G * d) + kh * d;
+            float y[PT], ss = 0.f;
+#pragma unroll
+            for (int p = 0; p < PT; ++p) {
+                y[p] = i0 + 128 * p < d ? conv(base + i0 + 128 * p) : 0.f;
+                ss = fmaf(y[p], y[p], ss);
             }
             ss = wave_sum(ss);
             if (lane == 0) red[wave] = ss;
-            if (tid < LQ_COLS) vs[tid] = j0 + tid < e ? conv(2 * a.G * d + h * e + j0 + tid) : 0.f;
-            if (tid == 0) bs[0] = dl_sigmoid(a.proj[(size_t)sg.row0 * a.ldp + a.b_off + h]);
-            if (a.channel) { for (int i = tid; i < d; i += 256) gs[i] = expf(an * a.ldec[((size_t)sg.row0 * a.H + h) * d + i]); }
-            else {
-                const float g = expf(an * dl_softplus(a.proj[(size_t)sg.row0 * a.ldp + a.a_off + h] + a.dt_bias[h]));
-                for (int i = tid; i < d; i += 256) gs[i] = g;
-            }
+            if (tid < LQ_COLS) vs[0][tid] = j0 + tid < e ? conv(2 * a.G * d + h * e + j0 + tid) : 0.f;
+            if (tid == 64) bs[0] = dl_sigmoid(a.proj[(size_t)sg.row0 * a.ldp + a.b_off + h]);
+            float gh = 0.f;
+            if (!a.channel) gh = expf(an * dl_softplus(a.proj[(size_t)sg.row0 * a.ldp + a.a_off + h] + a.dt_bias[h]));
+            for (int i = tid; i < ROWS; i += 256)
+                qkg[0][i][2] = i < d ? (a.channel ? expf(an * dl_softplus(a.ldec[((size_t)sg.row0 * a.H + h) * d + i])) : gh) : 0.f;
             __syncthreads();
-            const float fq = 1.f / (sqrtf(red[0] + red[1] + UNIT_EPS) * sqrtf((float)d)), fk = 1.f / sqrtf(red[2] + red[3] + UNIT_EPS);
-            for (int i = tid; i < d; i += 256) { qs[i] *= fq; ks[i] *= fk; }
+            const float f = wave < 2 ? 1.f / (sqrtf(red[0] + red[1] + UNIT_EPS) * sqrtf((float)d)) : 1.f / sqrtf(red[2] + red[3] + UNIT_EPS);
+#pragma unroll
+            for (int p = 0; p < PT; ++p)
+                if (i0 + 128 * p < ROWS) qkg[0][i0 + 128 * p][wave < 2 ? 0 : 1] = y[p] * f;
         } else {
-            for (int idx = tid; idx < nt * d; idx += 256) {
-                const int t = idx / d, i = idx - t * d;
+            for (int idx = tid; idx < nt * ROWS; idx += 256) {
+                const int t = idx / ROWS, i = idx % ROWS;
                 const size_t row = (size_t)(sg.row0 + t0 + t);
-                qs[idx] = a.xb[row * C + kh * d + i];
-                ks[idx] = a.xb[row * C + (a.G + kh) * d + i];
-                gs[idx] = expf(a.channel ? an * a.ldec[(row * a.H + h) * d + i] : a.ldec[row * a.H + h]);
+                f32x4 v = {0.f, 0.f, 0.f, 0.f};
+                if (i < d) {
+                    v[0] = a.xb[row * C + kh * d + i];
+                    v[1] = a.xb[row * C + (a.G + kh) * d + i];
+                    v[2] = expf(a.channel ? an * dl_softplus(a.ldec[(row * a.H + h) * d + i]) : a.ldec[row * a.H + h]);
+                }
+                qkg[t][i] = v;
             }
             for (int idx = tid; idx < nt * LQ_COLS; idx += 256) {
                 const int t = idx / LQ_COLS, c = j0 + idx % LQ_COLS;
-                vs[idx] = c < e ? a.xb[(size_t)(sg.row0 + t0 + t) * C + 2 * a.G * d + h * e + c] : 0.f;
+                vs[t][idx % LQ_COLS] = c < e ? a.xb[(size_t)(sg.row0 + t0 + t) * C + 2 * a.G * d + h * e + c] : 0.f;
             }
             for (int t = tid; t < nt; t += 256) bs[t] = a.beta[(size_t)(sg.row0 + t0 + t) * a.H + h];
         }
         __syncthreads();
         for (int t = 0; t < nt; ++t) {
-            const float *q = qs + t * d, *k = ks + t * d, *g = gs + t * d;
-            float p = 0.f, r = 0.f, kq = 0.f;
+            float p = 0.f, r = 0.f, kq = 0.f, k[NR];
 #pragma unroll
             for (int i = 0; i < NR; ++i) {
-                const int row = rg + LQ_GRP * i;
-                if (row < d) {
-                    S[i] *= g[row];
-                    p = fmaf(S[i], k[row], p);
-                    r = fmaf(S[i], q[row], r);
-                    kq = fmaf(k[row], q[row], kq);
-                }
+                const f32x4 c = qkg[t][rg + LQ_GRP * i];
+                S[i] *= c[2];
+                k[i] = c[1];
+                p = fmaf(S[i], c[1], p);
+                r = fmaf(S[i], c[0], r);
+                kq = fmaf(c[1], c[0], kq);
             }
-            float* pt = part + (t & 1) * LQ_GRP * LQ_COLS * 2;
-            pt[(rg * LQ_COLS + j) * 2] = p;
-            pt[(rg * LQ_COLS + j) * 2 + 1] = r;
-            float* kqs = red + 4 + (t & 1) * LQ_GRP;
-            if (j == 0) kqs[rg] = kq;
+            part[t & 1][rg][j][0] = p;
+            part[t & 1][rg][j][1] = r;
+            if (j == 0) kqs[t & 1][rg] = kq;
             __syncthreads();
             p = r = kq = 0.f;
 #pragma unroll
-            for (int x = 0; x < LQ_GRP; ++x) { p += pt[(x * LQ_COLS + j) * 2]; r += pt[(x * LQ_COLS + j) * 2 + 1]; kq += kqs[x]; }
-            const float u = bs[t] * (vs[t * LQ_COLS + j] - p);
+            for (int x = 0; x < LQ_GRP; ++x) { p += part[t & 1][x][j][0]; r += part[t & 1][x][j][1]; kq += kqs[t & 1][x]; }
+            const float u = bs[t] * (vs[t][j] - p);
 #pragma unroll
-            for (int i = 0; i < NR; ++i) {
-                const int row = rg + LQ_GRP * i;
-                if (row < d) S[i] = fmaf(k[row], u, S[i]);
-            }
+            for (int i = 0; i < NR; ++i) S[i] = fmaf(k[i], u, S[i]);
             if (rg == 0 && ok) a.o_raw[(size_t)(sg.row0 + t0 + t) * a.H * e + (size_t)h * e + col] = fmaf(kq, u, r);
         }
     }
@@ -273,7 +291,6 @@ __global__ __launch_bounds__(256) void lay_delta_seq_kernel(LDeltaArgs a, int ma
         for (int i = 0; i < NR; ++i) { const int row = rg + LQ_GRP * i; if (row < d) st[(size_t)row * e] = S[i]; }
     }
 }
-static size_t lay_delta_seq_lds(int d, int tb) { return (size_t)(3 * tb * d + tb * LQ_COLS + tb + 2 * LQ_GRP * LQ_COLS * 2 + 4 + 2 * LQ_GRP) * sizeof(float); }
 
 // head norm and output gate of the rows that went token by token, a wave per (row, head); TAIL (decode steps): blocks past the heads shift
 // the convolution's tail
@@ -297,7 +314,7 @@ __global__ __launch_bounds__(256) void lay_delta_out_kernel(LDeltaArgs a, int ma
     for (int c = lane; c < e; c += 64) ss = fmaf(o[c], o[c], ss);
     const float rs = 1.f / sqrtf(wave_sum(ss) / (float)e + a.eps);
     for (int c = lane; c < e; c += 64)
-        a.out[((size_t)r * a.H + h) * e + c] = o[c] * rs * a.norm_w[c] * a.gate[(size_t)r * a.ldg + (size_t)h * e + c];
+        a.out[((size_t)r * a.H + h) * e + c] = o[c] * rs * a.norm_w[c] * dl_gate(a.gate[(size_t)r * a.ldg + (size_t)h * e + c], a.gate_act);
 }
 
 // ------------------------------------------------------------------------------------------------------------------
@@ -352,7 +369,7 @@ __global__ __launch_bounds__(512) void lay_delta_chunk_prep_kernel(LDeltaArgs a)
         const float* x = a.xb + (size_t)(row0 + (in ? t : 0)) * C + kh * d + (in ? i : 0);
         Qs[t][i] = in ? x[0] : 0.f;
         Ks[t][i] = in ? x[a.G * d] : 0.f;
-        if (CH) Bs[t][i] = in ? fmaxf(an * a.ldec[((size_t)(row0 + t) * a.H + h) * d + i], LN_FLOOR) : 0.f;
+        if (CH) Bs[t][i] = in ? fmaxf(an * dl_softplus(a.ldec[((size_t)(row0 + t) * a.H + h) * d + i]), LN_FLOOR) : 0.f;
     }
     for (int idx = tid; idx < 2 * DC * DCP; idx += 512) (&Am[0][0])[idx] = 0.f;
     if (wave == 0) {
@@ -647,7 +664,8 @@ __global__ __launch_bounds__(256) void lay_delta_chunk_out_kernel(LDeltaArgs a) 
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int t = 16 * wave + 4 * kq + i;
-                if (t < n) a.out[((size_t)(row0 + t) * a.H + h) * e + col] = acc[m][i] * ss[i] * w * a.gate[(size_t)(row0 + t) * a.ldg + (size_t)h * e + col];
+                if (t < n)
+                    a.out[((size_t)(row0 + t) * a.H + h) * e + col] = acc[m][i] * ss[i] * w * dl_gate(a.gate[(size_t)(row0 + t) * a.ldg + (size_t)h * e + col], a.gate_act);
             }
         }
     }
@@ -659,7 +677,7 @@ __global__ __launch_bounds__(256) void lay_delta_chunk_out_kernel(LDeltaArgs a) 
 template <bool FUSED, int NR>
 static void lay_delta_seq_go(const LDeltaArgs& a, int max_n, hipStream_t s) {
     hipLaunchKernelGGL((lay_delta_seq_kernel<FUSED, NR>), dim3((unsigned)a.nseg, (unsigned)a.H, (unsigned)((a.e + LQ_COLS - 1) / LQ_COLS)), dim3(256),
-                       lay_delta_seq_lds(a.d, FUSED ? 1 : LAY_DELTA_SEQ), s, a, max_n);
+                       0, s, a, max_n);
 }
 template <bool FUSED>
 static void lay_delta_seq(const LDeltaArgs& a, int max_n, hipStream_t s) {
@@ -709,8 +727,10 @@ void launch_lay_delta(const LDeltaArgs& a, hipStream_t s) {
     launch_lay_conv_tail(c, a.nseg, s);
     const bool chunked = a.chunks && a.nchunks > 0 && a.scratch && lay_delta_chunk_fits(a.d, a.e);
     const int max_n = chunked ? LAY_DELTA_SEQ : 0x7fffffff;
-    lay_delta_seq<false>(a, max_n, s);
-    hipLaunchKernelGGL(lay_delta_out_kernel<false>, dim3((unsigned)a.T, (unsigned)head_blocks), dim3(256), 0, s, a, max_n, head_blocks);
+    if (a.min_n <= max_n) {
+        lay_delta_seq<false>(a, max_n, s);
+        hipLaunchKernelGGL(lay_delta_out_kernel<false>, dim3((unsigned)a.T, (unsigned)head_blocks), dim3(256), 0, s, a, max_n, head_blocks);
+    }
     if (!chunked) return;
     if (a.channel) { if (a.d <= 64) lay_delta_chunked<true, 64>(a, s); else lay_delta_chunked<true, 128>(a, s); }
     else { if (a.d <= 64) lay_delta_chunked<false, 64>(a, s); else lay_delta_chunked<false, 128>(a, s); }

@@ -49,10 +49,53 @@ __global__ __launch_bounds__(256) void lay_add_gnorm_kernel(float* __restrict__ 
     __syncthreads();
     for (int c = tid; c < W; c += 256) out[(size_t)r * W + c] = xr[c] * rs[c / gw] * w[c];
 }
+// one part, rows of up to 256 EPT elements: the row stays in registers between the update and the norm
+template <int EPT>
+__global__ __launch_bounds__(256) void lay_add_norm_reg_kernel(float* __restrict__ x, const int32_t* __restrict__ rows, const float* __restrict__ y,
+                                                               int nsum, const float* __restrict__ wsel, const float* __restrict__ w,
+                                                               float* __restrict__ out, int W, float eps) {
+    __shared__ float red[4];
+    const int r = blockIdx.x, tid = threadIdx.x;
+    float* xr = x + (size_t)(rows ? rows[r] : r) * W;
+    float v[EPT], nw[EPT];
+#pragma unroll
+    for (int i = 0; i < EPT; ++i) {
+        const int c = tid + 256 * i;
+        v[i] = c < W ? xr[c] : 0.f;
+        nw[i] = out && c < W ? w[c] : 0.f;
+    }
+    if (y) {
+        for (int k = 0; k < nsum; ++k) {
+            const float f = wsel ? wsel[(size_t)r * nsum + k] : 1.f;
+#pragma unroll
+            for (int i = 0; i < EPT; ++i) {
+                const int c = tid + 256 * i;
+                if (c < W) v[i] = fmaf(f, y[((size_t)r * nsum + k) * W + c], v[i]);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < EPT; ++i) if (tid + 256 * i < W) xr[tid + 256 * i] = v[i];
+        if (!out) return;
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < EPT; ++i) ss = fmaf(v[i], v[i], ss);
+    ss = wave_sum(ss);
+    if ((tid & 63) == 0) red[tid >> 6] = ss;
+    __syncthreads();
+    const float rs = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)W + eps);
+#pragma unroll
+    for (int i = 0; i < EPT; ++i) if (tid + 256 * i < W) out[(size_t)r * W + tid + 256 * i] = v[i] * rs * nw[i];
+}
 void launch_lay_add_gnorm(float* x, const int32_t* rows, const float* y, int nsum, const float* w, float* out, int n_rows, int W, int groups,
                           float eps, hipStream_t s, const float* wsel) {
     if (n_rows <= 0 || (!y && !out)) return;
     if (groups <= 0 || groups > LGN_MAX_GROUPS || W % groups) groups = 1;       // the configuration reader has refused these
+    if (groups == 1 && W <= 2048) {
+        if (W <= 1024) hipLaunchKernelGGL(lay_add_norm_reg_kernel<4>, dim3((unsigned)n_rows), dim3(256), 0, s, x, rows, y, nsum, wsel, w, out, W, eps);
+        else hipLaunchKernelGGL(lay_add_norm_reg_kernel<8>, dim3((unsigned)n_rows), dim3(256), 0, s, x, rows, y, nsum, wsel, w, out, W, eps);
+        return;
+    }
     hipLaunchKernelGGL(lay_add_gnorm_kernel, dim3((unsigned)n_rows), dim3(256), 0, s, x, rows, y, nsum, wsel, w, out, W, groups, eps);
 }
 

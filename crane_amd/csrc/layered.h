@@ -46,8 +46,8 @@ enum { LMIX_ATTN = 0, LMIX_LIGHTNING = 1, LMIX_LATENT = 2, LMIX_GLA = 3, LMIX_ME
 enum { LMLP_NONE = 0, LMLP_DENSE = 1, LMLP_MOE = 2 };
 // LACT_RELU2: max(v, 0)^2;  LACT_LOGSIG: act_param * ln(sigmoid(v)) (the logarithm of a decay sigmoid(v)^act_param)
 // LACT_CAPGLU (two-matrix products only): g = min(g, cap), u = clamp(u, -cap, cap): g sigmoid(1.702 g) (u + 1), cap = act_param
-// LACT_SOFTPLUS: ln(1 + e^v);  LACT_SOFTCAP: act_param * tanh(v / act_param)
-enum { LACT_NONE = 0, LACT_SILU = 1, LACT_SIGMOID = 2, LACT_GELU_TANH = 3, LACT_RELU2 = 4, LACT_LOGSIG = 5, LACT_CAPGLU = 6, LACT_SOFTPLUS = 7, LACT_SOFTCAP = 8 };
+// LACT_SOFTCAP: act_param * tanh(v / act_param)
+enum { LACT_NONE = 0, LACT_SILU = 1, LACT_SIGMOID = 2, LACT_GELU_TANH = 3, LACT_RELU2 = 4, LACT_LOGSIG = 5, LACT_CAPGLU = 6, LACT_SOFTCAP = 7 };
 // distance term taken off an attention score: none | r1 ln(1 + r2 (i - j)) | r1 (i - j)
 enum { LBIAS_NONE = 0, LBIAS_LOG = 1, LBIAS_LINEAR = 2 };
 // gate on the attention output: none | one value per head at g_off + head | one per element at g_off + head e + i
@@ -361,17 +361,18 @@ struct LDeltaArgs {
     int H, G, d, e;                                  // heads, query / key heads, key size, value size
     const float* conv_w; int taps;                   // [2 G d + H e][taps]
     float* conv_pool; size_t conv_stride, cv_off;    // tails [taps - 1][channels], oldest first
-    const float *dt_bias, *a_neg;                    // head form: ln g = a_neg[h] softplus(a + dt_bias[h]);  channel: ln g = a_neg[h] ldec
+    const float *dt_bias, *a_neg;                    // head form: ln g = a_neg[h] softplus(a + dt_bias[h]);  channel: ln g = a_neg[h] softplus(ldec)
     float* xb;                                       // [T][2 G d + H e]: convolved q (unit length, times d^(-1/2)) | k (unit length) | v
     float* beta;                                     // [T][H]
-    float* ldec; bool channel;                       // [T][H] (written by the preparation), or [T][H d] (channel: softplus already applied)
+    float* ldec; bool channel;                       // [T][H] (written by the preparation: ln g), or [T][H d] (channel: the argument of the softplus)
     float* state_pool; size_t slot_stride, st_off;
     const LaySegDev* segs; const int32_t* rowseg; int nseg, T;
-    const float* gate; int ldg;                      // activated output gate [T][H e]
+    const float* gate; int ldg, gate_act;            // output gate [T][H e] before its activation (LACT_SILU, LACT_SIGMOID)
     const float* norm_w; float eps;
     float* o_raw;                                    // [T][H e] scratch (token-by-token form)
     float* out;                                      // [T][H e]
     bool all_single;                                 // every portion of the pass is one token
+    int min_n;                                       // the shortest portion
     // chunk-parallel form for portions of more than LAY_DELTA_SEQ tokens: table {segment, first token}, segs[].pad1 = a segment's first
     // chunk; scratch of lay_delta_chunk_floats per (chunk, head).  Null / 0: every portion token by token.
     const int2* chunks = nullptr; int nchunks = 0; float* scratch = nullptr;

@@ -38,7 +38,7 @@ struct Layered {
     std::string arch;
     int max_conv = 0;                  // widest convolution of a state-space mixer or delta rule (channels)
     int max_gt = 0;
-    float* GT = nullptr;               // [cap][max_gt] activated output gates from a low-rank pair
+    float* GT = nullptr;               // [cap][max_gt] output gates from a low-rank pair
     float* DS = nullptr;               // delta rules, chunk-parallel form: ds_chunks chunks of ds_stride floats
     size_t ds_stride = 0;
     int ds_chunks = 0;
@@ -1452,7 +1452,7 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
         int32_t* t_wrows = tab + o; const size_t o_wrows = o; o += (size_t)T;
         LaySegDev* t_segs = (LaySegDev*)(tab + o); const size_t o_segs = o; o += (size_t)nseg * (sizeof(LaySegDev) / 4);
         int32_t* t_bt = tab + o; const size_t o_bt = o; o += (size_t)nseg * max_pages_per_seq;
-        int nw = 0, row = 0, nchunks = 0, dchunks = 0, max_n = 0;
+        int nw = 0, row = 0, nchunks = 0, dchunks = 0, max_n = 0, min_n = 0x7fffffff;
         long long max_len = 0;
         bool all_decode = true;
         for (int k = 0; k < nseg; ++k) {
@@ -1464,6 +1464,7 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
             nchunks += (n + LAY_LIGHT_CHUNK - 1) / LAY_LIGHT_CHUNK;
             if (n > LAY_DELTA_SEQ) dchunks += (n + LAY_DELTA_CHUNK - 1) / LAY_DELTA_CHUNK;
             max_n = std::max(max_n, n);
+            min_n = std::min(min_n, n);
             max_len = std::max(max_len, (long long)sp + n);
             memcpy(t_bt + (size_t)k * max_pages_per_seq, q.pages.data(), q.pages.size() * sizeof(int32_t));
             for (size_t pz = q.pages.size(); pz < (size_t)max_pages_per_seq; ++pz) t_bt[(size_t)k * max_pages_per_seq + pz] = 0;
@@ -1630,16 +1631,15 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
             a.state_pool = state_pool; a.slot_stride = state_slot_elems; a.st_off = w.st_off;
             a.segs = d_segs; a.rowseg = d_rowseg; a.nseg = nseg; a.T = T;
             a.gate = L.P + w.g_off; a.ldg = w.in_rows; a.norm_w = w.mix_norm; a.eps = cfg.eps;
-            a.o_raw = L.O; a.out = L.O2; a.all_single = all_decode;
+            a.gate_act = sp.channel_decay ? LACT_SIGMOID : LACT_SILU;
+            a.o_raw = L.O; a.out = L.O2; a.all_single = all_decode; a.min_n = min_n;
             if (dchunks > 0) { a.chunks = (const int2*)(L.d_tab + o_dchunks); a.nchunks = dchunks; a.scratch = L.DS; }
-            if (sp.channel_decay) {            // softplus of the decay's low-rank pair, sigmoid of the gate's
+            if (sp.channel_decay) {            // second halves of the two low-rank pairs
                 LGemmArgs gd;
                 gd.A = L.P + w.a_off; gd.lda = w.in_rows; gd.W = w.a2; gd.bias = w.dt_bias; gd.C = L.LD; gd.ldc = H * d; gd.M = T; gd.N = H * d; gd.K = sp.a_rank;
-                gd.act = LACT_SOFTPLUS; gd.act_split = gd.N;
                 lay_gemm(*this, L, gd, 1, s);
                 LGemmArgs gg;
                 gg.A = L.P + w.g_off; gg.lda = w.in_rows; gg.W = w.g2; gg.C = L.GT; gg.ldc = H * e; gg.M = T; gg.N = H * e; gg.K = sp.g_rank;
-                gg.act = LACT_SIGMOID; gg.act_split = gg.N;
                 lay_gemm(*this, L, gg, 1, s);
                 a.gate = L.GT; a.ldg = H * e;
             }
@@ -1741,8 +1741,7 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
                 add_gnorm(w.norm1, L.Hc);
                 LGemmArgs g;
                 g.A = L.Hc; g.lda = W; g.W = w.in_w; g.bias = w.in_b; g.C = L.P; g.ldc = w.in_rows; g.M = T; g.N = w.in_rows; g.K = W;
-                g.act_split = w.g_off; g.act = sp.mixer == LMIX_HGRN ? LACT_SILU : LACT_NONE;
-                g.act2 = sp.mixer == LMIX_DELTA && !sp.channel_decay ? LACT_SILU : LACT_NONE;
+                g.act_split = w.g_off; g.act = sp.mixer == LMIX_HGRN ? LACT_SILU : LACT_NONE; g.act2 = LACT_NONE;
                 lay_gemm(*this, L, g, 1, s);
                 const float* oa = L.O;
                 int on = 0;
