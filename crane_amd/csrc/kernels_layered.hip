@@ -1185,7 +1185,7 @@ __global__ __launch_bounds__(256) void lay_attn_kernel(LAttnArgs a) {
         return;
     }
     if (!qvalid) return;
-    const float* gp = a.proj + (size_t)row * a.ldp + a.g_off + (a.gate == LGATE_ELEM ? head * e : head);
+    const float* gp = a.gbuf + (size_t)row * a.ldg + (a.gate == LGATE_ELEM ? head * e : head);
     const float inv = (a.gate == LGATE_HEAD ? gp[0] : 1.f) / l * a.out_scale;
 #pragma unroll
     for (int c = 0; c < NACC; ++c) {
@@ -1399,7 +1399,7 @@ __global__ __launch_bounds__(LM_NT) void lay_attn_mfma_kernel(LAttnArgs a) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         if (!qok[r]) continue;
-        const float* gp = a.proj + (size_t)qrow[r] * a.ldp + a.g_off + (a.gate == LGATE_ELEM ? qhead[r] * e : qhead[r]);
+        const float* gp = a.gbuf + (size_t)qrow[r] * a.ldg + (a.gate == LGATE_ELEM ? qhead[r] * e : qhead[r]);
         const float inv = (a.gate == LGATE_HEAD ? gp[0] : 1.f) / l[r] * a.out_scale;
 #pragma unroll
         for (int n = 0; n < NEMAX; ++n)
@@ -1426,6 +1426,7 @@ static void lay_attn_mfma_go(const LAttnArgs& a, size_t lds, hipStream_t s) {
 void launch_lay_attn_mfma(const LAttnArgs& a0, hipStream_t s) {
     if (a0.ntiles <= 0) return;
     LAttnArgs a = a0;
+    if (!a.gbuf) { a.gbuf = a.proj + a.g_off; a.ldg = a.ldp; }
     if (a.e <= 0) a.e = a.d;
     const size_t pbytes = (size_t)2 * LM_NW * 16 * (LM_KT + 8);
     if (a.d <= 128 && a.e <= 128) {
@@ -1460,7 +1461,7 @@ __global__ __launch_bounds__(256) void lay_attn_merge_kernel(LAttnArgs a, int ns
             L = fmaf(a.part_ml[pr * 2 + 1], w, L);
             acc = fmaf(a.part_o[pr * d + i], w, acc);
         }
-        const float gate = a.gate == LGATE_NONE ? 1.f : a.proj[(size_t)row * a.ldp + a.g_off + (a.gate == LGATE_ELEM ? head * d + i : head)];
+        const float gate = a.gate == LGATE_NONE ? 1.f : a.gbuf[(size_t)row * a.ldg + (a.gate == LGATE_ELEM ? head * d + i : head)];
         a.out[(size_t)row * a.ldo + head * d + i] = acc * gate / L * a.out_scale;
     }
 }
@@ -1486,6 +1487,7 @@ static void lay_attn_go(const LAttnArgs& a, dim3 grid, size_t lds, hipStream_t s
 void launch_lay_attn(const LAttnArgs& a0, int kvt, hipStream_t s) {
     if (a0.ntiles <= 0) return;
     LAttnArgs a = a0;
+    if (!a.gbuf) { a.gbuf = a.proj + a.g_off; a.ldg = a.ldp; }
     if (a.e <= 0) a.e = a.d;               // values = whole key rows
     const bool own_v = a.vpool != nullptr;
     const int nsplit = (a.part_o && a.part_ml && a.nsplit > 1) ? a.nsplit : 1;
@@ -1946,11 +1948,11 @@ void launch_lay_memory_out(const float* o, const float* mrun, const float* gate,
 // ------------------------------------------------------------------------------------------------------------------
 // mixture of experts: router + counting sort
 // ------------------------------------------------------------------------------------------------------------------
-// One wave turns the E logits of token t in zs into choices and weights.  zs: [E] logits, then choice scores; sc = zs + E: [E] scores,
-// [groups], [top].
+// One wave turns the E logits of token t in zs into choices and weights.  zs: [E] logits, then choice scores (shared_gate: one more
+// logit behind them); sc: [E] scores, [groups], [top].
 __device__ __forceinline__ void lay_router_choose(float* zs, int t, int lane, int32_t* __restrict__ sel, float* __restrict__ wsel, int E, int top,
                                                   const RouterSpec& rs, const float* __restrict__ correction, int slots) {
-    float* sc = zs + E;
+    float* sc = zs + E + (rs.shared_gate ? 1 : 0);
     // wave 0: lane l owns outputs l, l + 64, ...; maxima, sums and the arg-max (lowest index among equals) are wave reductions
     auto arg_best = [&](bool want_max, int lo, int hi, float& bv) {      // over the live (not -inf) entries of zs[lo, hi)
         float v = 0.f; int at = 0x7fffffff;
@@ -2027,7 +2029,7 @@ __device__ __forceinline__ void lay_router_choose(float* zs, int t, int lane, in
         __builtin_amdgcn_wave_barrier();
     }
     for (int k = lane; k < top; k += 64) wsel[(size_t)t * slots + k] = (rs.normalise ? wl[k] / (wsum + 1e-20f) : wl[k]) * rs.scale;
-    for (int k = top + lane; k < slots; k += 64) wsel[(size_t)t * slots + k] = 1.f;
+    for (int k = top + lane; k < slots; k += 64) wsel[(size_t)t * slots + k] = rs.shared_gate ? 1.f / (1.f + expf(-zs[E])) : 1.f;
 }
 // logits and choice in one launch, one block per token
 __global__ __launch_bounds__(256) void lay_router_kernel(const float* __restrict__ h, const uint16_t* __restrict__ wr, int32_t* __restrict__ sel,
@@ -2036,7 +2038,7 @@ __global__ __launch_bounds__(256) void lay_router_kernel(const float* __restrict
     extern __shared__ float zs[];
     const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const float* hr = h + (size_t)t * W;
-    for (int ex = wave; ex < E; ex += 4) {
+    for (int ex = wave; ex < E + (rs.shared_gate ? 1 : 0); ex += 4) {
         float s = 0.f;
         for (int i = lane; i < W; i += 64) s = fmaf(hr[i], bf16_to_f32(wr[(size_t)ex * W + i]), s);
         s = wave_sum(s);
@@ -2054,7 +2056,8 @@ __global__ __launch_bounds__(256) void lay_router_choose_kernel(const float* __r
     const int t = blockIdx.x * 4 + wave;
     if (t >= T) return;
     float* mine = zs + (size_t)wave * per_wave;
-    for (int ex = lane; ex < E; ex += 64) mine[ex] = z[(size_t)t * E + ex];
+    const int ldz = E + (rs.shared_gate ? 1 : 0);
+    for (int ex = lane; ex < ldz; ex += 64) mine[ex] = z[(size_t)t * ldz + ex];
     __builtin_amdgcn_wave_barrier();
     lay_router_choose(mine, t, lane, sel, wsel, E, top, rs, correction, slots);
 }
@@ -2062,16 +2065,17 @@ void launch_lay_router(const float* h, const uint16_t* wr, int32_t* sel, float* 
                        const RouterSpec* rs, const float* correction, int slots, float* zbuf) {
     if (T <= 0) return;
     const RouterSpec r = rs ? *rs : RouterSpec();
+    const int logits = E + (r.shared_gate ? 1 : 0);
     if (zbuf && T <= LV_MAXM) {            // decode steps: logits by the streaming row kernel in f32 (every wave busy), then the choice
         LGemmArgs g;
-        g.A = h; g.lda = W; g.W = wr; g.C = zbuf; g.ldc = E; g.M = T; g.N = E; g.K = W;
+        g.A = h; g.lda = W; g.W = wr; g.C = zbuf; g.ldc = logits; g.M = T; g.N = logits; g.K = W;
         launch_lgemm(g, false, 1, s);
-        const int per_wave = 2 * E + r.groups + top;
+        const int per_wave = logits + E + r.groups + top;
         hipLaunchKernelGGL(lay_router_choose_kernel, dim3((unsigned)((T + 3) / 4)), dim3(256), (size_t)4 * per_wave * sizeof(float), s, zbuf, sel, wsel,
                            T, E, top, r, r.correction ? correction : nullptr, slots > top ? slots : top, per_wave);
         return;
     }
-    hipLaunchKernelGGL(lay_router_kernel, dim3((unsigned)T), dim3(256), (size_t)(2 * E + r.groups + top) * sizeof(float), s, h, wr, sel, wsel, W, E, top, r,
+    hipLaunchKernelGGL(lay_router_kernel, dim3((unsigned)T), dim3(256), (size_t)(logits + E + r.groups + top) * sizeof(float), s, h, wr, sel, wsel, W, E, top, r,
                        r.correction ? correction : nullptr, slots > top ? slots : top);
 }
 

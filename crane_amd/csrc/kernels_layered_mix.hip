@@ -100,6 +100,250 @@ void launch_lay_add_gnorm(float* x, const int32_t* rows, const float* y, int nsu
 }
 
 // ------------------------------------------------------------------------------------------------------------------
+// residual update + norm without a statistic: every thread is on its own
+// ------------------------------------------------------------------------------------------------------------------
+template <int VEC>
+__global__ __launch_bounds__(256) void lay_add_tanh_norm_kernel(float* __restrict__ x, const int32_t* __restrict__ rows, const float* __restrict__ y,
+                                                                int nsum, const float* __restrict__ wsel, float mult, float alpha,
+                                                                const float* __restrict__ w, const float* __restrict__ b,
+                                                                float* __restrict__ out, int W) {
+    typedef float vec __attribute__((ext_vector_type(VEC)));
+    const int r = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * VEC;
+    if (c >= W) return;
+    float* xr = x + (size_t)(rows ? rows[r] : r) * W + c;
+    vec v = *(const vec*)xr;
+    vec nw = 0.f, nb = 0.f;
+    if (out) { nw = *(const vec*)(w + c); nb = *(const vec*)(b + c); }
+    if (y) {
+        vec sum = 0.f;
+#pragma unroll 4
+        for (int k = 0; k < nsum; ++k) {   // fixed order: the same sum in every schedule
+            const float f = wsel ? wsel[(size_t)r * nsum + k] : 1.f;
+            const vec yk = *(const vec*)(y + ((size_t)r * nsum + k) * W + c);
+#pragma unroll
+            for (int i = 0; i < VEC; ++i) sum[i] = fmaf(f, yk[i], sum[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) v[i] = fmaf(mult, sum[i], v[i]);
+        *(vec*)xr = v;
+        if (!out) return;
+    }
+    vec o;
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) o[i] = fmaf(tanhf(alpha * v[i]), nw[i], nb[i]);
+    *(vec*)(out + (size_t)r * W + c) = o;
+}
+void launch_lay_add_tanh_norm(float* x, const int32_t* rows, const float* y, int nsum, const float* wsel, float mult, float alpha, const float* w,
+                              const float* b, float* out, int n_rows, int W, hipStream_t s) {
+    if (n_rows <= 0 || (!y && !out)) return;
+    // few rows (decode steps): narrow accesses, so that the row is spread over more threads
+    const int vec = W % 4 == 0 && (n_rows > 32 || W > 8192) ? 4 : 1;
+    const dim3 grid((unsigned)n_rows, (unsigned)((W / vec + 255) / 256));
+    if (vec == 4) hipLaunchKernelGGL(lay_add_tanh_norm_kernel<4>, grid, dim3(256), 0, s, x, rows, y, nsum, wsel, mult, alpha, w, b, out, W);
+    else hipLaunchKernelGGL(lay_add_tanh_norm_kernel<1>, grid, dim3(256), 0, s, x, rows, y, nsum, wsel, mult, alpha, w, b, out, W);
+}
+
+// ------------------------------------------------------------------------------------------------------------------
+// q, k, v between projection and attention: convolution, rotation, unit root mean square per head, cache append.
+// blockIdx.x: rpb consecutive rows; blockIdx.y < nqk: 256 / L query or key heads, L lanes each (a power of two, at most a wave) that own
+// the head's pairs ln, ln + L, ...; the others: 512 value channels, two per thread.  The convolution's window (up to four taps) rolls in
+// registers from row to row; longer ones read their taps per row.
+// ------------------------------------------------------------------------------------------------------------------
+constexpr int LCQ_TAPS = 4;
+// the channel's inputs at row `local - back` of a portion: projection rows, then the sequence's tail, then nothing
+__device__ __forceinline__ float lcq_input(const LConvQkvArgs& a, const LaySegDev& sg, int C, int c, int local) {
+    if (local >= 0) return a.src[(size_t)(sg.row0 + local) * a.lds + a.off + c];
+    const int t = a.taps - 1 + local;
+    return t >= 0 ? a.conv_pool[(size_t)sg.slot * a.slot_stride + a.cv_off + (size_t)t * C + c] : 0.f;
+}
+// channels c0, c0 + 1 (two: c0 even and everything 8-byte aligned) at once
+__device__ __forceinline__ float2 lcq_input2(const LConvQkvArgs& a, const LaySegDev& sg, int C, int c, int local) {
+    if (local >= 0) return *(const float2*)(a.src + (size_t)(sg.row0 + local) * a.lds + a.off + c);
+    const int t = a.taps - 1 + local;
+    return t >= 0 ? *(const float2*)(a.conv_pool + (size_t)sg.slot * a.slot_stride + a.cv_off + (size_t)t * C + c) : make_float2(0.f, 0.f);
+}
+// One thread's two channels ca, cb (-1: absent) through the convolution, row by row.
+template <bool ROLL>
+struct LcqPair {
+    int ca, cb, C; bool wide;
+    float2 w[ROLL ? LCQ_TAPS : 1], win[ROLL ? LCQ_TAPS - 1 : 1];
+    __device__ __forceinline__ float2 fetch(const LConvQkvArgs& a, const LaySegDev& sg, int local) const {
+        if (wide) return lcq_input2(a, sg, C, ca, local);
+        return make_float2(ca >= 0 ? lcq_input(a, sg, C, ca, local) : 0.f, cb >= 0 ? lcq_input(a, sg, C, cb, local) : 0.f);
+    }
+    __device__ __forceinline__ void init(const LConvQkvArgs& a, int ca_, int cb_, int C_, bool wide_) {
+        ca = ca_; cb = cb_; C = C_; wide = wide_ && ca >= 0 && cb == ca + 1;
+        if (ROLL) {
+#pragma unroll
+            for (int j = 0; j < LCQ_TAPS; ++j) {         // taps in front of the first one: weight 0
+                const int t = j - (LCQ_TAPS - a.taps);
+                w[j].x = t >= 0 && ca >= 0 ? a.cw[(size_t)t * C + ca] : 0.f;
+                w[j].y = t >= 0 && cb >= 0 ? a.cw[(size_t)t * C + cb] : 0.f;
+            }
+        }
+    }
+    // fresh: the first row of this thread's walk or of a portion
+    __device__ __forceinline__ float2 row(const LConvQkvArgs& a, const LaySegDev& sg, int local, bool fresh) {
+        float2 acc = make_float2(0.f, 0.f);
+        if (ROLL) {
+            const float2 now = fetch(a, sg, local);
+            if (fresh) {
+#pragma unroll
+                for (int j = 0; j < LCQ_TAPS - 1; ++j) win[j] = j >= LCQ_TAPS - a.taps ? fetch(a, sg, local - (LCQ_TAPS - 1) + j) : make_float2(0.f, 0.f);
+            }
+#pragma unroll
+            for (int j = 0; j < LCQ_TAPS - 1; ++j) { acc.x = fmaf(w[j].x, win[j].x, acc.x); acc.y = fmaf(w[j].y, win[j].y, acc.y); }
+            acc.x = fmaf(w[LCQ_TAPS - 1].x, now.x, acc.x); acc.y = fmaf(w[LCQ_TAPS - 1].y, now.y, acc.y);
+#pragma unroll
+            for (int j = 0; j < LCQ_TAPS - 2; ++j) win[j] = win[j + 1];
+            win[LCQ_TAPS - 2] = now;
+        } else
+            for (int j = 0; j < a.taps; ++j) {
+                const float2 v = fetch(a, sg, local - (a.taps - 1) + j);
+                acc.x = fmaf(ca >= 0 ? a.cw[(size_t)j * C + ca] : 0.f, v.x, acc.x);
+                acc.y = fmaf(cb >= 0 ? a.cw[(size_t)j * C + cb] : 0.f, v.y, acc.y);
+            }
+        return acc;
+    }
+    // one-token portions: the channel's tail moves on by the row (after row(), by the thread that owns the channel)
+    __device__ __forceinline__ void shift_tail(const LConvQkvArgs& a, const LaySegDev& sg) const {
+        float* tail = a.conv_pool + (size_t)sg.slot * a.slot_stride + a.cv_off;
+        const int n = a.taps - 1;
+        if (ROLL) {
+#pragma unroll
+            for (int j = 0; j < LCQ_TAPS - 1; ++j) {
+                const int t = j - (LCQ_TAPS - 1 - n);
+                if (t >= 0 && ca >= 0) tail[(size_t)t * C + ca] = win[j].x;
+                if (t >= 0 && cb >= 0) tail[(size_t)t * C + cb] = win[j].y;
+            }
+        } else
+            for (int t = 0; t < n; ++t) {
+                if (ca >= 0) tail[(size_t)t * C + ca] = t + 1 < n ? tail[(size_t)(t + 1) * C + ca] : a.src[(size_t)sg.row0 * a.lds + a.off + ca];
+                if (cb >= 0) tail[(size_t)t * C + cb] = t + 1 < n ? tail[(size_t)(t + 1) * C + cb] : a.src[(size_t)sg.row0 * a.lds + a.off + cb];
+            }
+    }
+};
+template <int KVT>
+__device__ __forceinline__ void lcq_store(void* pool, size_t at, int i0, int i1, float v0, float v1, bool wide) {
+    if (KVT == KV_F32) {
+        float* p = (float*)pool + at;
+        if (wide && i1 == i0 + 1) *(float2*)(p + i0) = make_float2(v0, v1);
+        else { p[i0] = v0; if (i1 >= 0) p[i1] = v1; }
+    } else {
+        uint16_t* p = (uint16_t*)pool + at;
+        if (wide && i1 == i0 + 1) *(uint32_t*)(p + i0) = pack_bf16x2(v0, v1);
+        else { p[i0] = f32_to_bf16(v0); if (i1 >= 0) p[i1] = f32_to_bf16(v1); }
+    }
+}
+// PPL: pairs per lane.  wide: d, e and every offset and stride are even
+template <int KVT, int PPL, bool ROLL>
+__global__ __launch_bounds__(256) void lay_conv_qkv_kernel(LConvQkvArgs a, int nqk, int L, int rpb, bool wide) {
+    const int tid = threadIdx.x, r0 = blockIdx.x * rpb, r1 = min(r0 + rpb, a.T);
+    const int C = (a.H + a.G) * a.d + a.G * a.e;
+    int seg = -1;
+    LaySegDev sg{};
+    if ((int)blockIdx.y >= nqk) {          // values
+        const int i0 = (((int)blockIdx.y - nqk) * 256 + tid) * 2, n = a.G * a.e;
+        if (i0 >= n) return;
+        const int i1 = i0 + 1 < n ? i0 + 1 : -1, base = (a.H + a.G) * a.d;
+        LcqPair<ROLL> pr;
+        pr.init(a, base + i0, i1 >= 0 ? base + i1 : -1, C, wide);
+        const int g0 = i0 / a.e, g1 = i1 >= 0 ? i1 / a.e : g0;
+        for (int r = r0; r < r1; ++r) {
+            const int sn = a.rowseg[r];
+            const bool fresh = sn != seg;
+            if (fresh) { sg = a.segs[sn]; seg = sn; }
+            const int local = r - sg.row0, pos = sg.start_pos + local;
+            const float2 v = pr.row(a, sg, local, fresh);
+            if (a.tail_too) pr.shift_tail(a, sg);
+            const size_t row = (size_t)a.bt[sg.bt_off + pos / a.page] * a.G * a.page + (size_t)(pos % a.page);
+            const size_t at0 = (row + (size_t)g0 * a.page) * a.e;
+            if (g0 == g1) lcq_store<KVT>(a.vpool, at0, i0 - g0 * a.e, i1 >= 0 ? i1 - g0 * a.e : -1, v.x, v.y, wide);
+            else {                         // (e odd) the pair lies in two heads
+                lcq_store<KVT>(a.vpool, at0, i0 - g0 * a.e, -1, v.x, 0.f, false);
+                lcq_store<KVT>(a.vpool, (row + (size_t)g1 * a.page) * a.e, i1 - g1 * a.e, -1, v.y, 0.f, false);
+            }
+        }
+        return;
+    }
+    const int hv = (int)blockIdx.y * (256 / L) + tid / L, ln = tid & (L - 1);
+    const bool live = hv < a.H + a.G;      // (dead lanes walk along: the shuffles below need whole waves)
+    const bool isq = hv < a.H;
+    const int hd = a.dims / 2, np = hd + (a.d - a.dims + 1) / 2;
+    LcqPair<ROLL> pr[PPL];
+    int e0[PPL], e1[PPL]; float fr[PPL];
+#pragma unroll
+    for (int p = 0; p < PPL; ++p) {        // a rotated pair, or two neighbours behind the rotated part (the last one may be alone)
+        const int i = ln + p * L;
+        e0[p] = e1[p] = -1; fr[p] = 0.f;
+        if (live && i < np) {
+            if (i < hd) { e0[p] = a.half ? i : 2 * i; e1[p] = a.half ? i + hd : 2 * i + 1; fr[p] = a.freq[i]; }
+            else { e0[p] = a.dims + 2 * (i - hd); e1[p] = e0[p] + 1 < a.d ? e0[p] + 1 : -1; }
+        }
+        pr[p].init(a, e0[p] >= 0 ? hv * a.d + e0[p] : -1, e1[p] >= 0 ? hv * a.d + e1[p] : -1, C, wide);
+    }
+    for (int r = r0; r < r1; ++r) {
+        const int sn = a.rowseg[r];
+        const bool fresh = sn != seg;
+        if (fresh) { sg = a.segs[sn]; seg = sn; }
+        const int local = r - sg.row0, pos = sg.start_pos + local;
+        float2 v[PPL];
+        float ss = 0.f;
+#pragma unroll
+        for (int p = 0; p < PPL; ++p) {
+            v[p] = pr[p].row(a, sg, local, fresh);
+            if (a.tail_too) pr[p].shift_tail(a, sg);
+            if (ln + p * L < hd) {
+                float sn_, cs;
+                sincosf((float)pos * fr[p], &sn_, &cs);
+                sn_ *= a.mag; cs *= a.mag;
+                v[p] = make_float2(v[p].x * cs - v[p].y * sn_, v[p].y * cs + v[p].x * sn_);
+            }
+            ss = fmaf(v[p].x, v[p].x, ss); ss = fmaf(v[p].y, v[p].y, ss);
+        }
+        float rs = 1.f;
+        if (a.unit) {
+            for (int o = L >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
+            rs = 1.f / sqrtf(ss / (float)a.d + a.eps);
+        }
+        const size_t krow = isq ? 0 : (((size_t)a.bt[sg.bt_off + pos / a.page] * a.G + (hv - a.H)) * a.page + (size_t)(pos % a.page)) * a.d;
+#pragma unroll
+        for (int p = 0; p < PPL; ++p) {
+            if (e0[p] < 0) continue;
+            if (isq) lcq_store<KV_F32>(a.q, (size_t)r * a.ldq + (size_t)hv * a.d, e0[p], e1[p], v[p].x * rs, v[p].y * rs, wide);
+            else lcq_store<KVT>(a.kpool, krow, e0[p], e1[p], v[p].x * rs, v[p].y * rs, wide);
+        }
+    }
+}
+template <int KVT>
+static void lay_conv_qkv_go(const LConvQkvArgs& a, dim3 grid, int nqk, int L, int ppl, int rpb, bool wide, hipStream_t s) {
+    const bool roll = a.taps <= LCQ_TAPS;
+    if (ppl <= 1) {
+        if (roll) hipLaunchKernelGGL((lay_conv_qkv_kernel<KVT, 1, true>), grid, dim3(256), 0, s, a, nqk, L, rpb, wide);
+        else hipLaunchKernelGGL((lay_conv_qkv_kernel<KVT, 1, false>), grid, dim3(256), 0, s, a, nqk, L, rpb, wide);
+    } else if (ppl <= 2) {
+        if (roll) hipLaunchKernelGGL((lay_conv_qkv_kernel<KVT, 2, true>), grid, dim3(256), 0, s, a, nqk, L, rpb, wide);
+        else hipLaunchKernelGGL((lay_conv_qkv_kernel<KVT, 2, false>), grid, dim3(256), 0, s, a, nqk, L, rpb, wide);
+    } else hipLaunchKernelGGL((lay_conv_qkv_kernel<KVT, 8, false>), grid, dim3(256), 0, s, a, nqk, L, rpb, wide);
+}
+void launch_lay_conv_qkv(const LConvQkvArgs& a0, int kvt, hipStream_t s) {
+    if (a0.T <= 0 || a0.H <= 0 || a0.d > LAY_CONV_QKV_MAX_DIM || a0.taps < 1) return;      // the configuration reader has refused these
+    LConvQkvArgs a = a0;
+    if (!a.freq) a.dims = 0;
+    const int np = a.dims / 2 + (a.d - a.dims + 1) / 2;
+    int L = 1;
+    while (L < np && L < 64) L <<= 1;
+    const int ppl = (np + L - 1) / L;
+    const int nqk = ((a.H + a.G) * L + 255) / 256, nv = (a.G * a.e + 511) / 512;
+    // decode steps: a block per row; prompt passes: the window rolls over a few rows
+    const int rpb = a.tail_too || a.T < 64 ? 1 : 8;
+    const bool wide = !((size_t)a.d & 1) && !((size_t)a.e & 1) && !(((size_t)a.lds | (size_t)a.off | (size_t)a.ldq | a.slot_stride | a.cv_off) & 1);
+    const dim3 grid((unsigned)((a.T + rpb - 1) / rpb), (unsigned)(nqk + (a.G > 0 ? nv : 0)));
+    if (kvt == KV_F32) lay_conv_qkv_go<KV_F32>(a, grid, nqk, L, ppl, rpb, wide, s);
+    else lay_conv_qkv_go<KV_BF16>(a, grid, nqk, L, ppl, rpb, wide, s);
+}
+
+// ------------------------------------------------------------------------------------------------------------------
 // two-map attention: one wave per (row, head)
 // ------------------------------------------------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void lay_diff_combine_kernel(const float* __restrict__ a, float* __restrict__ out, int T, int H, int G, int e,

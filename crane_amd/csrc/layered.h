@@ -28,6 +28,11 @@
 //     (S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q; short convolutions in front of q, k and v, unit-length q and k), one
 //     with a decay per head, one with a decay per key channel from a low-rank pair.  Capped gated feed-forwards, dense or routed
 //     (sigmoid scores, the best groups by the sum of their two largest scores, weights divided by their sum and scaled).
+//   Gizezen -- pre-norm layers with a scaled residual whose norms hold no statistic (tanh(alpha x) w + b element by element), a scaled
+//     embedding.  Sliding-window softmax attention with a short convolution on q, k and v behind their projections, interleaved rotation
+//     with banded stretching, unit root mean square per query / key head AFTER the rotation, one added to the softmax's denominator, a
+//     sigmoid gate per head, keys and values optionally borrowed from an earlier layer.  Mixture-of-experts feed-forwards whose weights
+//     are the softmax over the chosen logits, and a shared expert times a sigmoid of its own projection.
 // The mechanisms are kernels with their constants as arguments (kernels_layered.hip); the per-layer plumbing and the step function
 // over mixed batches (prompt portions beside single decode tokens) are in model_layered.cpp.
 #pragma once
@@ -75,6 +80,7 @@ struct RouterSpec {
     bool normalise = false;            // weights divided by their sum
     float scale = 1.f;                 // ... then times this
     int identity = 0;                  // the last `identity` outputs pass the input through (no matrices)
+    bool shared_gate = false;          // one more logit behind the outputs': its sigmoid is the weight of the expert every token uses
 };
 
 // one entry of config "layers"
@@ -109,7 +115,9 @@ struct LayerSpec {
     float qt_coef = 0.f; long long qt_every = 0;   // attention: q times 1 + qt_coef ln(floor((p + 1) / qt_every) + 1) at position p (0: off)
     bool talk = false;                 // attention: the heads' scores are mixed by a matrix [H][H] before mask and softmax
     bool head_norm = false;            // attention: RMS norm of every query (key) head by itself, one weight vector [dim] for all heads
+    bool unit_qk = false;              // attention: every query and key head over its own root mean square AFTER the rotation, no weight
     // state-space mixer: state size per head, groups of heads that share keys (B) and queries (C), convolution taps, parts of the output norm
+    // (attention: conv > 0: taps of the convolution on q, k and v behind their projections)
     int state = 0, groups = 1, conv = 0, norm_groups = 1;
     bool scale_input = false;          // mixture of experts: the expert's weight multiplies its input (false: its output)
     int expert_act = LACT_SILU; float limit = 0.f, shared_limit = 0.f;    // experts: activation of the gated product and its cap
@@ -122,6 +130,7 @@ struct LayerSpec {
 // device-side weights of one layer (bf16 matrices [out, in], f32 vectors)
 struct LayeredLayerW {
     float *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr;
+    float *norm1_off = nullptr, *norm2_off = nullptr; float norm1_alpha = 0.f, norm2_alpha = 0.f;     // tanh norms: offset vector, factor inside
     float *canon1 = nullptr, *canon2 = nullptr;      // [W][taps]
     // mixer input projection, rows concatenated so that one GEMM produces them:
     //   attention: q (H d) | k (G d) | g (H);  lightning: q (H d) | k (H d) | v (H e) | g (H e)
@@ -163,6 +172,7 @@ struct LayeredLayerW {
     float *conv_w = nullptr, *conv_b = nullptr, *dt_bias = nullptr, *a_neg = nullptr, *skip = nullptr;
     int z_off = 0, x_off = 0, dt_off = 0;
     size_t cv_off = 0;                               // the convolution's last taps - 1 inputs inside a slot of the conv pool (floats)
+    float* conv_wt = nullptr;                        // attention with a convolution on q | k | v: [taps][channels]
     // delta rule: columns of the projection row: q_off: q | k | v (the convolution's channels) | b_off (write strength) | a_off (decay per head, or
     // a1) | g_off (gate, or g1);  a2: [H d][a_rank], g2: [H e][g_rank];  conv_w, dt_bias ([H] or [H d]), a_neg ([H]), mix_norm ([e])
     int b_off = 0;
@@ -235,6 +245,7 @@ void launch_lay_post_norm(float* x, const float* y, const float* w, float mult, 
 
 struct LAttnArgs {
     const float* proj; int ldp, q_off, g_off;        // activated projection rows: q | k | gate
+    const float* gbuf = nullptr; int ldg = 0;        // gates in rows of their own (null: proj + g_off, rows of ldp)
     float* out; int ldo;                             // [T][H d], gated
     const void* kpool;                               // [n_pages][G][page][d]
     const int32_t* bt; const LaySegDev* segs; const int2* tiles; int ntiles;
@@ -311,6 +322,28 @@ void launch_lay_rms_gate(const float* o, const float* gate, int ldg, const float
                          int group = 0, bool shared_w = false);
 
 // ---- kernels_layered_mix.hip ----
+// norm without a statistic: x[r] += mult * sum_(k < nsum) y[(r nsum + k) W ..] (y null: nothing is added; wsel given: row k times
+// wsel[r nsum + k]), then out[r][c] = tanh(alpha x[rows ? rows[r] : r][c]) w[c] + b[c] (out null: the update alone).  rows and y exclude each other.
+void launch_lay_add_tanh_norm(float* x, const int32_t* rows, const float* y, int nsum, const float* wsel, float mult, float alpha, const float* w,
+                              const float* b, float* out, int n_rows, int W, hipStream_t s);
+// queries, keys and values of a pass between their projection and attention, one launch: causal convolution per channel (tails as in
+// LConvArgs), then on query and key heads the rotation by position and -- unit -- division by the head's root mean square; q -> rows of
+// their own, keys and values -> the sequence's pages.  G = 0: queries alone (keys and values are another layer's).
+struct LConvQkvArgs {
+    const float* src; int lds, off;                  // projection rows: q (H d) | k (G d) | v (G e) from column off: the convolution's channels
+    int H, G, d, e;
+    const float* cw; int taps;                       // [taps][channels], the last row the current token's
+    float* conv_pool; size_t slot_stride, cv_off;    // tails [taps - 1][channels], oldest first
+    int dims; bool half; const float* freq; float mag;   // rotation (freq null: none), as lay_rope
+    bool unit; float eps;
+    float* q; int ldq;                               // [T][H d]
+    void *kpool, *vpool;                             // [n_pages][G][page][d] / [e]
+    const int32_t* bt; const LaySegDev* segs; const int32_t* rowseg; int page, T;
+    bool tail_too = false;                           // every portion of the pass is one token: a channel's tail is shifted by its thread
+                                                     // (otherwise launch_lay_conv_tail follows)
+};
+constexpr int LAY_CONV_QKV_MAX_DIM = 1024;           // largest d
+void launch_lay_conv_qkv(const LConvQkvArgs& a, int kvt, hipStream_t s);
 // x[r] += sum_(k < nsum) y[(r nsum + k) W ..] (y null: nothing is added; wsel given: row k times wsel[r nsum + k]), then out[r] =
 // x[rows ? rows[r] : r] in `groups` equal consecutive parts, each over its own root mean square, times w (out null: the update alone).
 // rows and y exclude each other.
@@ -384,7 +417,8 @@ void launch_lay_delta(const LDeltaArgs& a, hipStream_t s);
 
 // router: z = h . Wr^T in f32 over E outputs, scores by rs (sigmoid of each / softmax over all), the `top` largest choice scores
 // (score + correction, inside the best groups; lowest index first among equals) -> sel [T top], wsel [T slots] = their scores
-// (normalised when asked); slots > top: the remaining weights are 1 (rows that every token uses, e.g. a shared expert)
+// (normalised when asked); slots > top: the remaining weights are 1 (rows that every token uses, e.g. a shared expert), or the sigmoid
+// of logit E (rs.shared_gate: wr has E + 1 rows and zbuf E + 1 columns)
 // zbuf [T][E] given and few rows (decode steps): the logits come from the streaming row kernel (f32 products of the unrounded rows),
 // then one wave per token chooses; otherwise one block per token does both
 void launch_lay_router(const float* h, const uint16_t* wr, int32_t* sel, float* wsel, int T, int W, int E, int top, hipStream_t s,

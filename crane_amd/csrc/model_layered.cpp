@@ -30,9 +30,10 @@ struct Layered {
     // Gibipel: a sublayer reads the residual itself and a one-number norm sits on its output; embedding and logits are scaled
     bool post_only = false;
     float embed_scale = 1.f, logit_scale = 1.f;
-    // Nevotar, Rirotar: x += mixer(norm1 x), x += ff(norm2 x).  Nevotar's norms work on norm_groups equal parts of the vector and its
-    // logits come from the embedding table; Rirotar's logits pass logit_cap tanh(z / logit_cap)
-    bool pre_norm = false;
+    // Nevotar, Rirotar, Gizezen: x += mult mixer(norm1 x), x += mult ff(norm2 x).  Nevotar's norms work on norm_groups equal parts of the
+    // vector and its logits come from the embedding table; Rirotar's logits pass logit_cap tanh(z / logit_cap); Gizezen's norms are
+    // tanh(alpha x) w + b element by element (tanh_norm), mult is a constant of its configuration (1 for the other two)
+    bool pre_norm = false, tanh_norm = false;
     int norm_groups = 1;
     float logit_cap = 0.f;
     std::string arch;
@@ -48,7 +49,7 @@ struct Layered {
     float *KM = nullptr, *MR = nullptr, *HS = nullptr;   // matrix memory: key factor and running maximum per token and head; shared expert's inner rows
     int max_q = 0, max_qa = 0, max_cq = 0, max_ld = 0, max_e = 0;
     bool f32 = false;                  // number format of the projections and the key cache
-    float* final_norm = nullptr;
+    float *final_norm = nullptr, *final_off = nullptr; float final_alpha = 0.f;
     uint16_t* head = nullptr;
     int cap = 0;                       // rows of one pass
     int max_in = 0, max_o = 0, max_ff = 0, max_top = 1, max_E = 1;
@@ -266,6 +267,24 @@ static void parse_mononex_layer(const cmjson::Value& e, LayerSpec& sp, const std
     sp.gated_ff = false; sp.ff_act = LACT_RELU2;
 }
 
+// "rot": {"base", "dims", "scaling": {"factor", "low", "high", "original"}}, the scaling in bands of wavelengths; half: pairs (i, i + dims / 2)
+static void parse_rotation(const cmjson::Value* rt, LayerSpec& a, bool half) {
+    if (!rt || rt->kind != cmjson::Value::Obj) return;
+    a.rot.half = half;
+    a.rot.dims = (int)rt->integer("dims", a.dim);
+    a.rot.base = rt->number("base", 10000.0);
+    if (const cmjson::Value* sc = rt->get("scaling"))
+        if (sc->kind == cmjson::Value::Obj) {
+            a.rot.banded = true;
+            a.rot.factor = sc->number("factor", 1.0);
+            a.rot.low = sc->number("low", 1.0);
+            a.rot.high = sc->number("high", 4.0);
+            a.rot.original = sc->number("original", 0.0);
+            need(a.rot.factor > 0 && a.rot.original > 0 && a.rot.low > 0 && a.rot.high > a.rot.low, "rot.scaling");
+        }
+    need(a.rot.dims >= 0 && a.rot.dims <= a.dim && a.rot.dims % 2 == 0 && a.rot.base > 1.0, "rot.dims / rot.base");
+}
+
 // Gibipel: layer type "parallel" = "mixer": {"left": window attention with pooled blocks, "right": matrix memory, "left_scale",
 // "right_scale"}; "mlp": mixture of experts with a softmax router ("identity", "groups": {"count", "keep"}, tensor "correction") and
 // an optional "shared" expert
@@ -295,22 +314,7 @@ static void parse_gibipel_layer(const cmjson::Value& e, LayerSpec& sp) {
                 a.pool = mk->integer("pool", 0);
                 need(a.win > 0 && a.pool >= 0, "mask.size / mask.pool");
             }
-        if (const cmjson::Value* rt = lf->get("rot"))
-            if (rt->kind == cmjson::Value::Obj) {
-                a.rot.half = true;
-                a.rot.dims = (int)rt->integer("dims", a.dim);
-                a.rot.base = rt->number("base", 10000.0);
-                if (const cmjson::Value* sc = rt->get("scaling"))
-                    if (sc->kind == cmjson::Value::Obj) {
-                        a.rot.banded = true;
-                        a.rot.factor = sc->number("factor", 1.0);
-                        a.rot.low = sc->number("low", 1.0);
-                        a.rot.high = sc->number("high", 4.0);
-                        a.rot.original = sc->number("original", 0.0);
-                        need(a.rot.factor > 0 && a.rot.original > 0 && a.rot.low > 0 && a.rot.high > a.rot.low, "rot.scaling");
-                    }
-                need(a.rot.dims >= 0 && a.rot.dims <= a.dim && a.rot.dims % 2 == 0 && a.rot.base > 1.0, "rot.dims / rot.base");
-            }
+        parse_rotation(lf->get("rot"), a, true);
         a.bias = LBIAS_NONE; a.gate = LGATE_NONE; a.sink = true; a.own_v = true; a.qk_norm = true; a.qkv_bias = true;
         need(lay_attn_fits(a.dim, a.vdim, true), "attention head sizes too large");
     }
@@ -330,7 +334,7 @@ static void parse_gibipel_layer(const cmjson::Value& e, LayerSpec& sp) {
     sp.router.softmax = true; sp.router.correction = true; sp.router.normalise = true;
 }
 
-// softmax attention sizes shared by Nevotar's two attention kinds
+// softmax attention sizes shared by Nevotar's two attention kinds and Gizezen's
 static void parse_attn_sizes(const cmjson::Value& mx, LayerSpec& a) {
     a.mixer = LMIX_ATTN;
     a.heads = (int)mx.integer("heads", 0);
@@ -476,27 +480,68 @@ static void parse_rirotar_layer(const cmjson::Value& e, LayerSpec& sp) {
     sp.router.group_top = 2; sp.router.normalise = true;
 }
 
+// Gizezen: layer type "attention" ("heads", "kv_heads", "dim", "vdim", "conv", "scale", "mask": {"size"}, "rot": {"base", "dims", "scaling":
+// {"factor", "low", "high", "original"}}, optional "kv_from"); "mlp": {"kind": "moe", "expert": {"ff"}, "router": {"experts", "top"},
+// "shared": {"ff"}} or null
+static void parse_gizezen_layer(const cmjson::Value& e, LayerSpec& sp, const std::vector<LayerSpec>& before) {
+    const std::string type = e.string("type", "");
+    if (type != "attention") throw CmError(CM_ERR_UNSUPPORTED, "layer type '" + type + "' not implemented");
+    const cmjson::Value* mx = e.get("mixer");
+    need(mx && mx->kind == cmjson::Value::Obj, "layer without mixer");
+    parse_attn_sizes(*mx, sp);
+    sp.qkv_bias = false; sp.gate = LGATE_HEAD; sp.sink = true; sp.unit_qk = true;
+    sp.conv = (int)mx->integer("conv", 1);
+    need(sp.conv >= 1 && sp.conv <= 64, "conv");
+    if (const cmjson::Value* mk = mx->get("mask"))
+        if (mk->kind == cmjson::Value::Obj) {
+            sp.win = mk->integer("size", sp.win);
+            need(sp.win > 0, "mask.size");
+        }
+    parse_rotation(mx->get("rot"), sp, false);
+    if (const cmjson::Value* kf = mx->get("kv_from"))
+        if (kf->kind == cmjson::Value::Num) {
+            sp.kv_from = (int)kf->num;
+            need(sp.kv_from >= 0 && sp.kv_from < (int)before.size(), "kv_from names no earlier layer");
+            const LayerSpec& src = before[(size_t)sp.kv_from];
+            need(src.mixer == LMIX_ATTN && src.kv_from < 0 && src.kv_heads == sp.kv_heads && src.dim == sp.dim && src.vdim == sp.vdim,
+                 "kv_from: the other layer's keys and values do not fit");
+        }
+    need(sp.dim <= LAY_CONV_QKV_MAX_DIM && lay_attn_fits(sp.dim, sp.vdim, true), "attention head sizes too large");
+    const cmjson::Value* ml = e.get("mlp");
+    if (ml && ml->kind == cmjson::Value::Obj) {
+        need(ml->string("kind", "moe") == "moe", "mlp.kind: only 'moe'");
+        parse_mlp(ml, sp, true);
+        need(sp.router.identity == 0 && sp.router.groups == 1 && sp.router.scale == 1.f && sp.limit == 0.f && sp.shared_limit == 0.f,
+             "router.identity / groups / scale and expert limits are not part of this design");
+        // softmax over the chosen logits = softmax over all of them, divided by the chosen ones' sum
+        sp.router.softmax = true; sp.router.normalise = true; sp.router.shared_gate = sp.shared_ff > 0;
+    }
+}
+
 // config.json of a layer-list decoder: "architecture", "vocab", "width", "norm".eps and "layers": [{"type", "mixer": {...}, "mlp"}]
 void Model::init_layered_config(const cmjson::Value& root) {
     const std::string arch = root.string("architecture", "");
-    const char* known[] = {"Korupel", "Mononex", "Gibipel", "Nevotar", "Rirotar"};
+    const char* known[] = {"Korupel", "Mononex", "Gibipel", "Nevotar", "Rirotar", "Gizezen"};
     if (std::find(std::begin(known), std::end(known), arch) == std::end(known))
-        throw CmError(CM_ERR_UNSUPPORTED, "architecture '" + arch + "' not implemented (Korupel, Mononex, Gibipel, Nevotar, Rirotar)");
+        throw CmError(CM_ERR_UNSUPPORTED, "architecture '" + arch + "' not implemented (Korupel, Mononex, Gibipel, Nevotar, Rirotar, Gizezen)");
     layered = true;
     lay.reset(new Layered());
     Layered& L = *lay;
     L.arch = arch;
     L.parallel = arch == "Mononex";
     L.post_only = arch == "Gibipel";
-    L.pre_norm = arch == "Nevotar" || arch == "Rirotar";
+    L.tanh_norm = arch == "Gizezen";
+    L.pre_norm = arch == "Nevotar" || arch == "Rirotar" || L.tanh_norm;
     cfg.model_type = arch;
     for (char& c : cfg.model_type) c = (char)std::tolower((unsigned char)c);
     if (arch == "Rirotar") {
         L.logit_cap = (float)root.number("logit_softcap", 0.0);
         need(L.logit_cap > 0.f, "logit_softcap");
     }
-    if (L.post_only) {
+    if (L.post_only || L.tanh_norm)
         if (const cmjson::Value* em = root.get("embedding")) L.embed_scale = (float)em->number("scale", 1.0);
+    if (L.tanh_norm) L.mult = (float)root.number("residual_mult", 1.0);
+    if (L.post_only) {
         L.logit_scale = (float)root.number("logit_scale", 1.0);
     }
     cfg.V = (int)root.integer("vocab", 0);
@@ -520,6 +565,7 @@ void Model::init_layered_config(const cmjson::Value& root) {
         else if (L.post_only) parse_gibipel_layer(*e, sp);
         else if (arch == "Nevotar") parse_nevotar_layer(*e, sp, L.spec);
         else if (arch == "Rirotar") parse_rirotar_layer(*e, sp);
+        else if (L.tanh_norm) parse_gizezen_layer(*e, sp, L.spec);
         else parse_korupel_layer(*e, sp);
         L.spec.push_back(sp);
     }
@@ -647,6 +693,7 @@ static void build_mononex(Model& m, LaySource& src);
 static void build_gibipel(Model& m, LaySource& src);
 static void build_nevotar(Model& m, LaySource& src);
 static void build_rirotar(Model& m, LaySource& src);
+static void build_gizezen(Model& m, LaySource& src);
 
 static void build_layered(Model& m, LaySource& src) {
     Layered& L = *m.lay;
@@ -654,6 +701,7 @@ static void build_layered(Model& m, LaySource& src) {
     if (L.post_only) { build_gibipel(m, src); return; }
     if (L.arch == "Nevotar") { build_nevotar(m, src); return; }
     if (L.arch == "Rirotar") { build_rirotar(m, src); return; }
+    if (L.tanh_norm) { build_gizezen(m, src); return; }
     const size_t W = (size_t)m.cfg.H, V = (size_t)m.cfg.V;
     const float ws = 1.0f / std::sqrt((float)W);
     m.embed = up_bf16(m, src.get("embed", V * W, 1.0f, 0.f));
@@ -827,7 +875,9 @@ static void build_experts(Model& m, LaySource& src, const std::string& p, const 
     }
     w.gate = up_bf16(m, g); w.up = up_bf16(m, u); w.down = up_bf16(m, dn);
     const size_t outs = (size_t)(sp.experts + sp.router.identity);
-    w.router = up_bf16(m, src.get(p + "mlp.router", outs * W, ws, 0.f));
+    std::vector<float> router = src.get(p + "mlp.router", outs * W, ws, 0.f);
+    if (sp.router.shared_gate) append(router, src.get(p + "mlp.shared.sg", W, ws, 0.f));
+    w.router = up_bf16(m, router);
     if (sp.router.correction) w.correction = up_f32(m, src.get(p + "mlp.correction", outs, 0.02f, 0.f));
     if (sp.shared_ff > 0) {
         const size_t sf = (size_t)sp.shared_ff;
@@ -1114,6 +1164,56 @@ static void build_rirotar(Model& m, LaySource& src) {
     m.lm_head = L.head;
 }
 
+static void build_gizezen(Model& m, LaySource& src) {
+    Layered& L = *m.lay;
+    const size_t W = (size_t)m.cfg.H, V = (size_t)m.cfg.V;
+    const float ws = 1.0f / std::sqrt((float)W);
+    m.embed = up_bf16(m, src.get("embed", V * W, 1.0f, 0.f));
+    auto norm = [&](const std::string& name, float*& w, float*& off, float& alpha) {
+        w = up_f32(m, src.get(name, W, 0.1f, 1.f));
+        off = up_f32(m, src.get(name + ".b", W, 0.1f, 0.f));
+        alpha = src.get(name + ".alpha", 1, 0.05f, 0.5f)[0];
+    };
+    L.w.resize(L.spec.size());
+    for (size_t i = 0; i < L.spec.size(); ++i) {
+        const LayerSpec& sp = L.spec[i];
+        LayeredLayerW& w = L.w[i];
+        const std::string p = "l" + std::to_string(i) + ".", q = p + "mix.";
+        const size_t H = (size_t)sp.heads, G = sp.kv_from >= 0 ? 0 : (size_t)sp.kv_heads, d = (size_t)sp.dim, e = (size_t)sp.vdim, taps = (size_t)sp.conv;
+        norm(p + "norm1", w.norm1, w.norm1_off, w.norm1_alpha);
+        // q | k | v | gate (keys and values borrowed: q | gate); the convolutions of q, k and v as one, tap by tap
+        const size_t C = (H + G) * d + G * e;
+        std::vector<float> in, ct(taps * C);
+        size_t c0 = 0;
+        for (const char* n : {"q", "k", "v"}) {
+            const size_t rows = *n == 'q' ? H * d : (*n == 'k' ? G * d : G * e);
+            if (rows == 0) continue;
+            append(in, src.get(q + n, rows * W, ws, 0.f));
+            const std::vector<float> cw = src.get(q + n + ".conv", rows * taps, 1.0f / std::sqrt((float)taps), 0.f);
+            for (size_t r = 0; r < rows; ++r)
+                for (size_t j = 0; j < taps; ++j) ct[j * C + c0 + r] = cw[r * taps + j];
+            c0 += rows;
+        }
+        w.conv_wt = up_f32(m, ct);
+        w.q_off = 0; w.k_off = (int)(H * d); w.v_off = (int)((H + G) * d); w.g_off = (int)C;
+        append(in, src.get(q + "g", H * W, ws, 0.f));
+        // whole tiles for the projection's kernels: rows of zeros behind the last one (their products are not read)
+        const size_t rows = in.size() / W, unit = rows >= 1024 ? 128 : 8;
+        w.in_rows = (int)((rows + unit - 1) / unit * unit);
+        in.resize((size_t)w.in_rows * W, 0.f);
+        w.in_w = up_bf16(m, in);
+        w.o_w = up_bf16(m, src.get(q + "o", W * H * e, 1.0f / std::sqrt((float)(H * e)), 0.f));
+        w.sink = up_f32(m, std::vector<float>(H, 0.f));       // one in the denominator: exp(0)
+        if (sp.rot.dims > 0) w.rot_freq = up_f32(m, rot_frequencies(sp.rot, &w.rot_mag));
+        if (sp.mlp == LMLP_NONE) continue;
+        norm(p + "norm2", w.norm2, w.norm2_off, w.norm2_alpha);
+        build_experts(m, src, p, sp, w);
+    }
+    norm("final.norm", L.final_norm, L.final_off, L.final_alpha);
+    L.head = up_bf16(m, src.get("head", V * W, ws, 0.f));
+    m.lm_head = L.head;
+}
+
 void load_layered_from_dir(Model& m, const std::string& dir) {
     try {
         LayFileSource src(dir);
@@ -1182,6 +1282,11 @@ void Model::alloc_runtime_layered() {
                 }
                 pool_bytes = (pool_bytes + 15) / 16 * 16;
             }
+            if (sp.mixer == LMIX_ATTN && sp.conv > 0) {       // the convolution's last taps - 1 inputs [taps - 1][q | k | v] (borrowed keys: [q])
+                w.cv_off = cv;
+                cv += (size_t)(sp.conv - 1) * (sp.heads * sp.dim + (sp.kv_from >= 0 ? 0 : sp.kv_heads * (sp.dim + sp.vdim)));
+                L.max_conv = std::max(L.max_conv, sp.heads * sp.dim);      // (the convolved queries)
+            }
             const int nrep = sp.heads / sp.kv_heads;
             if (std::find(L.nreps.begin(), L.nreps.end(), nrep) == L.nreps.end()) L.nreps.push_back(nrep);
             L.max_o = std::max(L.max_o, sp.heads * sp.maps * ev);
@@ -1247,7 +1352,7 @@ void Model::alloc_runtime_layered() {
         if (sp.mlp != LMLP_NONE) L.max_ff = std::max(L.max_ff, sp.ff);
         if (sp.mlp == LMLP_MOE) {
             L.max_top = std::max(L.max_top, sp.top);
-            L.max_E = std::max(L.max_E, sp.experts + sp.router.identity);
+            L.max_E = std::max(L.max_E, sp.experts + sp.router.identity + (sp.router.shared_gate ? 1 : 0));
             L.max_slots = std::max(L.max_slots, sp.top + (sp.shared_ff > 0 ? 1 : 0));
             L.max_sff = std::max(L.max_sff, sp.shared_ff);
         }
@@ -1552,9 +1657,9 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
         };
         // softmax attention of one layer over the pages: queries at qsrc[row ldq + q_off + head dk], output [T][H ev] into L.O
         auto run_attention = [&](const LayerSpec& sp, const LayeredLayerW& w, const float* qsrc, int ldq, int q_off, int g_off, int dk, int ev,
-                                 float* out = nullptr, int ldo = 0, float out_scale = 1.f, int v_div = 1) {
+                                 float* out = nullptr, int ldo = 0, float out_scale = 1.f, int v_div = 1, const float* gbuf = nullptr, int ldg = 0) {
             LAttnArgs a;
-            a.v_div = v_div;
+            a.v_div = v_div; a.gbuf = gbuf; a.ldg = ldg;
             a.proj = qsrc; a.ldp = ldq; a.q_off = q_off; a.g_off = g_off;
             a.out = out ? out : L.O; a.ldo = out ? ldo : sp.heads * ev; a.out_scale = out_scale;
             if (sp.pool > 0) {
@@ -1674,8 +1779,9 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
         };
         // pre-norm layers: the finished sublayer's rows (nsum per token, summed in order) join the residual inside the next norm's launch
         struct { const float* y = nullptr; int nsum = 1; const float* wsel = nullptr; } padd;
-        auto add_gnorm = [&](const float* nw_, float* out) {
-            launch_lay_add_gnorm(L.X, nullptr, padd.y, padd.nsum, nw_, out, T, W, L.norm_groups, cfg.eps, s, padd.wsel);
+        auto add_norm = [&](const float* nw_, const float* off, float alpha, float* out) {
+            if (L.tanh_norm) launch_lay_add_tanh_norm(L.X, nullptr, padd.y, padd.nsum, padd.wsel, L.mult, alpha, nw_, off, out, T, W, s);
+            else launch_lay_add_gnorm(L.X, nullptr, padd.y, padd.nsum, nw_, out, T, W, L.norm_groups, cfg.eps, s, padd.wsel);
             padd.y = nullptr; padd.wsel = nullptr;
         };
         const float *par_y1 = nullptr, *par_y2 = nullptr;       // parallel layers: sublayer outputs not yet added to the residual
@@ -1737,15 +1843,36 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
                     par_y1 = par_y2 = nullptr;
                 }
             } else if (L.pre_norm) {
-                // ---- x += mixer(norm1 x), x += ff(norm2 x), norms in equal parts
-                add_gnorm(w.norm1, L.Hc);
+                // ---- x += mult mixer(norm1 x), x += mult ff(norm2 x); norms in equal parts, or of single elements
+                add_norm(w.norm1, w.norm1_off, w.norm1_alpha, L.Hc);
                 LGemmArgs g;
                 g.A = L.Hc; g.lda = W; g.W = w.in_w; g.bias = w.in_b; g.C = L.P; g.ldc = w.in_rows; g.M = T; g.N = w.in_rows; g.K = W;
-                g.act_split = w.g_off; g.act = sp.mixer == LMIX_HGRN ? LACT_SILU : LACT_NONE; g.act2 = LACT_NONE;
+                g.act_split = w.g_off; g.act = sp.mixer == LMIX_HGRN ? LACT_SILU : LACT_NONE;
+                g.act2 = sp.mixer == LMIX_ATTN && sp.gate != LGATE_NONE ? LACT_SIGMOID : LACT_NONE;
                 lay_gemm(*this, L, g, 1, s);
                 const float* oa = L.O;
                 int on = 0;
-                if (sp.mixer == LMIX_ATTN) {
+                if (sp.mixer == LMIX_ATTN && sp.maps == 1) {
+                    // convolution, rotation, unit heads and cache append in one launch (queries into rows of their own), then attention over
+                    // the layer's pages or those of the layer it borrows from
+                    const int H = sp.heads, d = sp.dim, e = sp.vdim;
+                    LConvQkvArgs c;
+                    c.src = L.P; c.lds = w.in_rows; c.off = w.q_off; c.H = H; c.G = sp.kv_from >= 0 ? 0 : sp.kv_heads; c.d = d; c.e = e;
+                    c.cw = w.conv_wt; c.taps = sp.conv; c.conv_pool = conv_pool; c.slot_stride = conv_slot_elems; c.cv_off = w.cv_off;
+                    c.dims = sp.rot.dims; c.half = sp.rot.half; c.freq = w.rot_freq; c.mag = w.rot_mag; c.unit = sp.unit_qk; c.eps = cfg.eps;
+                    c.q = L.XB; c.ldq = H * d; c.kpool = kv_pool + w.k_pool_off; c.vpool = kv_pool + w.v_pool_off;
+                    c.bt = d_bt; c.segs = d_segs; c.rowseg = d_rowseg; c.page = page; c.T = T; c.tail_too = all_decode;
+                    launch_lay_conv_qkv(c, kv_mode, s);
+                    if (!all_decode && sp.conv > 1) {
+                        LConvArgs t;
+                        t.src = L.P; t.lds = w.in_rows; t.off = w.q_off; t.C = w.g_off; t.dst = nullptr; t.ldd = 0; t.cw = nullptr; t.cb = nullptr;
+                        t.taps = sp.conv; t.act = LACT_NONE; t.conv_pool = conv_pool; t.slot_stride = conv_slot_elems; t.cv_off = w.cv_off;
+                        t.segs = d_segs; t.rowseg = d_rowseg;
+                        launch_lay_conv_tail(t, nseg, s);
+                    }
+                    run_attention(sp, w, L.XB, H * d, 0, 0, d, e, nullptr, 0, 1.f, 1, L.P + w.g_off, w.in_rows);
+                    on = H * e;
+                } else if (sp.mixer == LMIX_ATTN) {
                     // two maps per head as heads of their own (2 H query heads over 2 G key heads, pairs of key heads share a value head)
                     const int H = sp.heads, G = sp.kv_heads, d = sp.dim, e = sp.vdim;
                     LQkPrepExtra ex;
@@ -1846,7 +1973,7 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
                 lay_gemm(*this, L, go, 1, s);
                 padd.y = L.Y; padd.nsum = 1;
                 if (sp.mlp == LMLP_DENSE) {
-                    add_gnorm(w.norm2, L.Hc);
+                    add_norm(w.norm2, w.norm2_off, w.norm2_alpha, L.Hc);
                     LGemmArgs gu;
                     gu.A = L.Hc; gu.lda = W; gu.W = w.gate; gu.W2 = w.up; gu.C = L.HH; gu.ldc = sp.ff; gu.M = T; gu.N = sp.ff; gu.K = W;
                     gu.act = sp.ff_act; gu.act_param = sp.limit;
@@ -1856,7 +1983,7 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
                     lay_gemm(*this, L, dn, 1, s);
                     padd.y = L.Y; padd.nsum = 1;
                 } else if (sp.mlp == LMLP_MOE) {
-                    add_gnorm(w.norm2, L.Hc);
+                    add_norm(w.norm2, w.norm2_off, w.norm2_alpha, L.Hc);
                     // scale_input: an expert's weight multiplies its INPUT, the rows of the grouped product are w h and the combine is a plain
                     // sum; otherwise the weights join in the combine
                     const int slots = sp.top + (sp.shared_ff > 0 ? 1 : 0);
@@ -1883,7 +2010,7 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
                     }
                     padd.y = L.YS; padd.nsum = slots; padd.wsel = sp.scale_input ? nullptr : L.wsel;
                 }
-                if (L.capture || li + 1 == L.spec.size()) add_gnorm(nullptr, nullptr);
+                if (L.capture || li + 1 == L.spec.size()) add_norm(nullptr, nullptr, 0.f, nullptr);
             } else if (L.post_only) {
                 // ---- the sublayers read the residual itself; x += g * unit(sublayer(x)).  All mixers of the layer share one input
                 // projection and one output projection (their heads side by side in its input, each times its scale)
@@ -2033,7 +2160,8 @@ void Model::step_batch(const StepItem* items, size_t n_items, float* logits_out,
         // ---- final norm + head over the wanted rows, LOGIT_ROWS at a time
         for (int w0 = 0; w0 < nw; w0 += Layered::LOGIT_ROWS) {
             const int nr = std::min(Layered::LOGIT_ROWS, nw - w0);
-            if (L.pre_norm) launch_lay_add_gnorm(L.X, d_wrows + w0, nullptr, 0, L.final_norm, L.Xw, nr, W, L.norm_groups, cfg.eps, s);
+            if (L.tanh_norm) launch_lay_add_tanh_norm(L.X, d_wrows + w0, nullptr, 0, nullptr, 0.f, L.final_alpha, L.final_norm, L.final_off, L.Xw, nr, W, s);
+            else if (L.pre_norm) launch_lay_add_gnorm(L.X, d_wrows + w0, nullptr, 0, L.final_norm, L.Xw, nr, W, L.norm_groups, cfg.eps, s);
             else launch_lay_rms_rows(L.X, d_wrows + w0, L.final_norm, L.Xw, nr, W, cfg.eps, s);
             LGemmArgs hd;
             hd.A = L.Xw; hd.lda = W; hd.W = L.head; hd.C = logitsb; hd.ldc = V; hd.M = nr; hd.N = V; hd.K = W;
@@ -2103,7 +2231,7 @@ uint64_t Model::layered_decode_bytes(size_t ctx) const {
         if (sp.mlp == LMLP_DENSE) b += (sp.gated_ff ? 6ull : 4ull) * W * sp.ff;
         else if (sp.mlp == LMLP_MOE) {
             const uint64_t real = (uint64_t)std::min(sp.top, sp.experts);
-            b += 6ull * W * sp.ff * real + 2ull * W * (sp.experts + sp.router.identity) + 6ull * W * sp.shared_ff;
+            b += 6ull * W * sp.ff * real + 2ull * W * (sp.experts + sp.router.identity + (sp.router.shared_gate ? 1 : 0)) + 6ull * W * sp.shared_ff;
         }
     }
     return b;
