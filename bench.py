@@ -146,7 +146,7 @@ def relaunch_under_torchrun(n: int) -> int:
 
 
 def korupel_leg(args, names=None, prompt_lens=None, label="korupel"):
-    """--korupel / --mononex / --gibipel / --nevotar / --rirotar: prompt and decode throughput of a layer-list decoder (crane_amd/csrc/model_layered.cpp)
+    """--korupel / --mononex / --gibipel / --nevotar / --rirotar / --gizezen: prompt and decode throughput of a layer-list decoder (crane_amd/csrc/model_layered.cpp)
     at the widths of a real model, random weights, beside the closest family of the library at equal size: the Qwen3.5 hybrid
     (linear attention 3 : 1 softmax attention, same width / ff / layers / vocabulary).  One JSON line; the default workload of this
     script is not touched."""
@@ -258,6 +258,9 @@ def main():
     ap.add_argument("--rirotar", default=None, metavar="CONFIGS", help="comma-separated registry configs (e.g. "
                     "rirotar-1b,mononex-1b,korupel-1b-moe,qwen3.5-0.8b): prompt and decode throughput of each instead of the headline workload")
     ap.add_argument("--rirotar-prompts", default="512,2048", help="prompt lengths of --rirotar")
+    ap.add_argument("--gizezen", default=None, metavar="CONFIGS", help="comma-separated registry configs (e.g. "
+                    "gizezen-1b,gibipel-1b,korupel-1b-moe or gizezen-8b-4l,gibipel-8b-4l): prompt and decode throughput of each instead of the headline workload")
+    ap.add_argument("--gizezen-prompts", default="512,2048", help="prompt lengths of --gizezen")
     ap.add_argument("--nevotar-prompts", default="512,2048", help="prompt lengths of --nevotar")
     args = ap.parse_args()
     if args.korupel:
@@ -268,6 +271,8 @@ def main():
         sys.exit(korupel_leg(args, args.gibipel, args.gibipel_prompts, "gibipel"))
     if args.rirotar:
         sys.exit(korupel_leg(args, args.rirotar, args.rirotar_prompts, "rirotar"))
+    if args.gizezen:
+        sys.exit(korupel_leg(args, args.gizezen, args.gizezen_prompts, "gizezen"))
     if args.nevotar:
         sys.exit(korupel_leg(args, args.nevotar, args.nevotar_prompts, "nevotar"))
 

@@ -355,6 +355,55 @@ CONFIGS.update({
 })
 
 
+# ---- layer-list decoders: Gizezen ------------------------------------------------------------------------------------------
+def gizezen_config(vocab: int, width: int, pattern: str, heads: int, kv_heads: int, dim: int, vdim: int, window: int, experts: int, top: int,
+                   expert_ff: int, shared_ff: int = 0, conv: int = 4, rot_dims: "int | None" = None, rot_base: float = 500000.0,
+                   scaling: "dict | None" = None, embed_scale: float = 1.0, residual_mult: float = 1.0, eps: float = 1e-6) -> dict:
+    """pattern: one letter per layer -- 'a' window attention with keys and values of its own, 'b' the same with those of the nearest 'a'
+    before it; upper case: no feed-forward (all others: a mixture of experts)."""
+    layers, last_a = [], None
+    for i, ch in enumerate(pattern):
+        rot = dict(base=rot_base, dims=dim if rot_dims is None else rot_dims)
+        if scaling:
+            rot["scaling"] = dict(scaling)
+        mixer = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, conv=conv, scale=dim ** -0.5, mask=dict(size=window), rot=rot)
+        if ch.lower() == "b":
+            if last_a is None:
+                raise ValueError("'b' needs an 'a' layer before it")
+            mixer["kv_from"] = last_a
+        elif ch.lower() == "a":
+            last_a = i
+        else:
+            raise ValueError(f"pattern letter {ch!r}")
+        mlp = None
+        if ch.islower():
+            mlp = dict(kind="moe", expert=dict(ff=expert_ff), router=dict(experts=experts, top=top))
+            if shared_ff:
+                mlp["shared"] = dict(ff=shared_ff)
+        layers.append(dict(type="attention", mixer=mixer, mlp=mlp))
+    return dict(architecture="Gizezen", vocab=vocab, width=width, norm=dict(eps=eps), embedding=dict(scale=embed_scale),
+                residual_mult=residual_mult, layers=layers)
+
+
+_GIZEZEN_1B = dict(heads=8, kv_heads=2, dim=128, vdim=128, window=1024, experts=14, top=4, expert_ff=768, shared_ff=512, scaling=_BANDS,
+                   residual_mult=0.25, embed_scale=4.0)
+CONFIGS.update({
+    "tiny-gizezen": gizezen_config(320, 128, "abAba", heads=4, kv_heads=2, dim=32, vdim=24, window=20, experts=6, top=2, expert_ff=48, shared_ff=64,
+                                   conv=3, rot_dims=16, rot_base=10000.0, scaling=dict(factor=2.0, low=1.0, high=4.0, original=64),
+                                   embed_scale=3.0, residual_mult=0.4),
+    # the widths of gibipel-1b / korupel-1b-moe (1024 wide, 24 layers, vocabulary 248 320, 8 query / 2 key heads of 128, window 1024), every
+    # second layer on the keys and values of the one before it; 14 experts of 768, 4 per token, and a shared expert of 512 (3584 active inner
+    # columns, as the dense models)
+    "gizezen-1b": gizezen_config(248320, 1024, "ab" * 12, **_GIZEZEN_1B),
+    "gizezen-1b-4l": gizezen_config(32768, 1024, "abab", **_GIZEZEN_1B),
+    # layers of an 8B-class model (4096 wide, 32 query / 8 key heads of 128), 4 of them
+    "gizezen-8b-4l": gizezen_config(32768, 4096, "abab", heads=32, kv_heads=8, dim=128, vdim=128, window=4096, experts=16, top=4, expert_ff=2048,
+                                    shared_ff=2048, scaling=_BANDS, residual_mult=0.25, embed_scale=4.0),
+    "gibipel-8b-4l": gibipel_config(32768, 4096, 4, heads=32, kv_heads=8, dim=128, vdim=128, window=4096, pool=64, mem_heads=32, mem_dim=64,
+                                    mem_vdim=128, experts=16, top=4, expert_ff=2048, shared_ff=2048, scaling=_BANDS, rot_base=500000.0),
+})
+
+
 def get_config(name: str) -> dict:
     if name not in CONFIGS:
         raise KeyError(f"unknown config {name!r}; have {sorted(CONFIGS)}")
