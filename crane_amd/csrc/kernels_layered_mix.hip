@@ -336,7 +336,7 @@ void launch_lay_conv_qkv(const LConvQkvArgs& a0, int kvt, hipStream_t s) {
     const int ppl = (np + L - 1) / L;
     const int nqk = ((a.H + a.G) * L + 255) / 256, nv = (a.G * a.e + 511) / 512;
     // decode steps: a block per row; prompt passes: the window rolls over a few rows
-    const int rpb = a.tail_too || a.T < 64 ? 1 : 8;
+    const int rpb = a.tail_too || a.T < 64 ? 1 : 4;
     const bool wide = !((size_t)a.d & 1) && !((size_t)a.e & 1) && !(((size_t)a.lds | (size_t)a.off | (size_t)a.ldq | a.slot_stride | a.cv_off) & 1);
     const dim3 grid((unsigned)((a.T + rpb - 1) / rpb), (unsigned)(nqk + (a.G > 0 ? nv : 0)));
     if (kvt == KV_F32) lay_conv_qkv_go<KV_F32>(a, grid, nqk, L, ppl, rpb, wide, s);
