@@ -43,16 +43,25 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
     return t;
 }
 
-// embedding rows of any width (the shared gather moves four elements at a time)
+// embedding rows of any width, times a factor
+template <int VEC>
 __global__ __launch_bounds__(256) void lay_embed_rows_kernel(const uint16_t* __restrict__ emb, const uint32_t* __restrict__ ids,
                                                              float* __restrict__ x, int W, int V, float scale) {
     uint32_t tok = ids[blockIdx.x];
     if (tok >= (uint32_t)V) tok = 0;
-    for (int i = threadIdx.x; i < W; i += 256) x[(size_t)blockIdx.x * W + i] = bf16_to_f32(emb[(size_t)tok * W + i]) * scale;
+    const int i = (blockIdx.y * 256 + threadIdx.x) * VEC;
+    if (i >= W) return;
+    const uint16_t* src = emb + (size_t)tok * W + i;
+    float* dst = x + (size_t)blockIdx.x * W + i;
+    if (VEC == 4) {
+        const u32x2 p = *(const u32x2*)src;
+        *(f32x4*)dst = (f32x4){bf16_lo(p[0]) * scale, bf16_hi(p[0]) * scale, bf16_lo(p[1]) * scale, bf16_hi(p[1]) * scale};
+    } else dst[0] = bf16_to_f32(src[0]) * scale;
 }
 void launch_lay_embed_rows(const uint16_t* emb, const uint32_t* ids, float* x, int T, int W, int V, hipStream_t s, float scale) {
     if (T <= 0) return;
-    hipLaunchKernelGGL(lay_embed_rows_kernel, dim3((unsigned)T), dim3(256), 0, s, emb, ids, x, W, V, scale);
+    if (W % 4 == 0) hipLaunchKernelGGL(lay_embed_rows_kernel<4>, dim3((unsigned)T, (unsigned)((W + 1023) / 1024)), dim3(256), 0, s, emb, ids, x, W, V, scale);
+    else hipLaunchKernelGGL(lay_embed_rows_kernel<1>, dim3((unsigned)T, (unsigned)((W + 255) / 256)), dim3(256), 0, s, emb, ids, x, W, V, scale);
 }
 
 // ------------------------------------------------------------------------------------------------------------------
